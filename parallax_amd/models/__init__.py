@@ -20,3 +20,4 @@ from . import vurizen  # noqa: F401
 from . import sogidra  # noqa: F401
 from . import zabusun  # noqa: F401
 from . import pudizen  # noqa: F401
+from . import runidra  # noqa: F401

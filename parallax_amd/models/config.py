@@ -17,6 +17,22 @@ from typing import Any, Dict, List, Optional
 # (no pooled rows, no recurrent state slots, no layer reading another's rows)
 _PLAIN_ROW_DESIGNS = ("Pudizen",)
 
+# layer-list designs whose config may run a range of layers several times
+# ('loop') over several copies of the residual stream ('streams')
+_LOOPED_DESIGNS = ("Runidra",)
+
+
+def feed_forward_kind(mlp: Dict[str, Any]) -> str:
+    """'moe' or 'dense' of a layer-list feed-forward entry: its 'kind', or by
+    whether it has a router."""
+    return mlp.get("kind", "moe" if "router" in mlp else "dense")
+
+
+def mlstm_state_width(dim: int, vdim: int) -> int:
+    """fp32 numbers one mLSTM head keeps per request: the [dim, vdim] matrix,
+    the [dim] normaliser and the running maximum, padded to 16 bytes."""
+    return (dim * vdim + dim + 1 + 3) // 4 * 4
+
 
 @dataclass
 class ModelConfig:
@@ -91,10 +107,16 @@ class ModelConfig:
     linear_value_head_dim: int = 0
     linear_conv_kernel_dim: int = 4
 
-    # -- per-layer stacks (vurizen, sogidra, zabusun, pudizen): every layer carries its own mixer and
+    # -- per-layer stacks (vurizen, sogidra, zabusun, pudizen, runidra): every layer carries its own mixer and
     # feed-forward description; the flat fields above hold the first layer's
     # values only so that sizing helpers have something to read ----------------
     layer_specs: Optional[List[Dict[str, Any]]] = None
+    # stacks that run some layers several times: entry i is a layer RUN (with a
+    # cache entry or state of its own) and layer_weights[i] the index of the
+    # layer whose tensors it uses; None: run i uses layer i's
+    layer_weights: Optional[List[int]] = None
+    streams: int = 1                 # copies of the residual stream (hyper-connections)
+    logit_softcap: float = 0.0       # > 0: logits <- cap * tanh(logits / cap)
     residual_mult: float = 1.0
     logit_scale: float = 1.0         # the logits are multiplied by this
     norm_groups: int = 1             # RMS norms split the width into this many parts
@@ -193,6 +215,9 @@ class ModelConfig:
                                           int(mx["vdim"]))))
                 elif sp["type"] == "parallel":   # the recurrent half: a vector
                     shapes.append(((0,), (int(mx["right"]["width"]),)))
+                elif sp["type"] == "mlstm":      # matrix, normaliser, maximum
+                    shapes.append(((0,), (int(mx["heads"]), mlstm_state_width(
+                        int(mx["dim"]), int(mx["vdim"])))))
             return shapes
         if not self.has_linear_layers:
             return []
@@ -217,7 +242,7 @@ class ModelConfig:
         """Whether any layer keeps recurrent state in a per-request slot."""
         if self.layer_specs is not None:
             return self.architecture not in _PLAIN_ROW_DESIGNS and any(
-                sp["type"] in ("gla", "parallel") for sp in self.layer_specs)
+                sp["type"] in ("gla", "parallel", "mlstm") for sp in self.layer_specs)
         return bool(self.layer_types) and "linear_attention" in self.layer_types
 
     def layer_type(self, layer_idx: int) -> str:
@@ -253,9 +278,14 @@ class ModelConfig:
         values), 'attention_2' (sliding window, sigmoid key weights),
         'latent_attention' (no positions, gated); its top level also carries
         'embedding' {"scale", "bigram": {"buckets", "mul_prev", "mul_cur"}}
-        and 'norm' {"eps", "groups"}."""
+        and 'norm' {"eps", "groups"}. Runidra has 'mlstm' and a
+        'latent_attention' with a query latent and sinks, and the top-level
+        keys 'streams', 'loop' {"start", "stop", "times"}, 'logit_scale' and
+        'logit_softcap'."""
         if cfg["architecture"] in _PLAIN_ROW_DESIGNS:
             return cls._from_plain_row_config(cfg)
+        if cfg["architecture"] in _LOOPED_DESIGNS:
+            return cls._from_looped_config(cfg)
         layers = cfg["layers"]
         kinds = {"gla": "linear_attention", "latent_attention": "latent_attention",
                  "attention": "diff_attention",
@@ -271,12 +301,8 @@ class ModelConfig:
         linear = [sp["mixer"] for sp in layers if sp["type"] == "gla"]
         windowed = [sp["mixer"] for sp in layers if sp["type"] == "attention_2"]
         mlps = [sp["mlp"] for sp in layers if sp.get("mlp") is not None]
-
-        def kind_of(m):   # a feed-forward without a router is a dense one
-            return m.get("kind", "moe" if "router" in m else "dense")
-
-        moes = [m for m in mlps if kind_of(m) == "moe"]
-        dense = [m for m in mlps if kind_of(m) == "dense"]
+        moes = [m for m in mlps if feed_forward_kind(m) == "moe"]
+        dense = [m for m in mlps if feed_forward_kind(m) == "dense"]
         first = layers[0]["mixer"]
         if layers[0]["type"] == "parallel":
             first = first["left"]
@@ -375,6 +401,82 @@ class ModelConfig:
         ffs = [int(sp["mlp"]["ff"]) for sp in layers if sp.get("mlp") is not None]
         if ffs:
             mc.intermediate_size = ffs[0]
+        return mc
+
+    @classmethod
+    def _from_looped_config(cls, cfg: Dict[str, Any]) -> "ModelConfig":
+        """Layers of 'mlstm' and 'latent_attention' mixers; layers start ..
+        stop - 1 of 'loop' run `times` times in a row. The result counts RUNS:
+        num_layers, layer_specs and layer_types have one entry per run, so
+        that cache geometry and layer ranges need no notion of a loop."""
+        layers = cfg["layers"]
+        kinds = {"mlstm": "linear_attention", "latent_attention": "latent_attention"}
+        for sp in layers:
+            if sp["type"] not in kinds:
+                raise ValueError(f"unknown layer type {sp['type']!r}")
+            mlp = sp.get("mlp")
+            if mlp is not None and feed_forward_kind(mlp) not in ("dense", "moe"):
+                raise ValueError(f"unknown feed-forward kind {mlp.get('kind')!r}")
+        loop = cfg.get("loop") or {}
+        start, stop = int(loop.get("start", 0)), int(loop.get("stop", 0))
+        times = int(loop.get("times", 1))
+        if not 0 <= start <= stop <= len(layers) or times < 1:
+            raise ValueError(f"loop {loop} does not fit {len(layers)} layers")
+        runs = (list(range(start)) + list(range(start, stop)) * times
+                + list(range(stop, len(layers))))
+        specs = [layers[i] for i in runs]
+        first = layers[0]["mixer"]
+        mc = cls(
+            architecture=cfg["architecture"],
+            model_type=str(cfg["architecture"]).lower(),
+            vocab_size=int(cfg["vocab"]),
+            hidden_size=int(cfg["width"]),
+            num_layers=len(runs),
+            num_heads=int(first["heads"]),
+            num_kv_heads=int(first["heads"]),
+            head_dim=int(first["dim"]),
+            rms_norm_eps=float(cfg["norm"]["eps"]),
+            max_position_embeddings=int(cfg.get("max_positions", 1 << 20)),
+            layer_types=[kinds[sp["type"]] for sp in specs],
+            eos_token_ids=[],
+            bos_token_id=None,
+            torch_dtype=cfg.get("torch_dtype", "bfloat16"),
+            layer_specs=specs,
+            layer_weights=runs,
+            streams=int(cfg.get("streams", 1)),
+            logit_scale=float(cfg.get("logit_scale", 1.0)),
+            logit_softcap=float(cfg.get("logit_softcap") or 0.0),
+            raw=cfg,
+        )
+        if mc.streams < 1:
+            raise ValueError("there is at least one residual stream")
+        latent = [sp["mixer"] for sp in layers if sp["type"] == "latent_attention"]
+        if latent:
+            mc.q_lora_rank = int(latent[0]["q_rank"])
+            mc.kv_lora_rank = int(latent[0]["kv_rank"])
+            mc.qk_nope_head_dim = int(latent[0]["dim"])
+            mc.qk_rope_head_dim = int(latent[0]["rot_dim"])
+            mc.v_head_dim = int(latent[0]["vdim"])
+            mc.sliding_window = int(latent[0]["mask"]["size"])
+        linear = [sp["mixer"] for sp in layers if sp["type"] == "mlstm"]
+        if linear:
+            mc.linear_num_key_heads = mc.linear_num_value_heads = int(linear[0]["heads"])
+            mc.linear_key_head_dim = int(linear[0]["dim"])
+            mc.linear_value_head_dim = int(linear[0]["vdim"])
+            mc.linear_conv_kernel_dim = 1
+        mlps = [sp["mlp"] for sp in layers if sp.get("mlp") is not None]
+        dense = [m for m in mlps if feed_forward_kind(m) == "dense"]
+        moes = [m for m in mlps if feed_forward_kind(m) == "moe"]
+        if dense:
+            mc.intermediate_size = int(dense[0]["ff"])
+        if moes:
+            mc.num_experts = int(moes[0]["router"]["experts"])
+            mc.num_experts_per_tok = int(moes[0]["router"]["top"])
+            mc.moe_intermediate_size = int(moes[0]["expert"]["ff"])
+            if moes[0].get("shared"):
+                mc.shared_expert_intermediate_size = int(moes[0]["shared"]["ff"])
+            if not dense:
+                mc.intermediate_size = mc.moe_intermediate_size
         return mc
 
     @classmethod

@@ -13,6 +13,11 @@ before it), separate W_uk / W_uv, rotate-half pairing on the first rot_dims
 dimensions of the rotated part with a YaRN frequency ramp whose softmax scale
 is left untouched, and a layer may read ANOTHER layer's cache rows
 (`cache_layer_idx` of the owner) with its own queries and up-projections.
+Switches: the queries may come through a latent of their own (`q_rank`: down
+projection, RMS norm, up projection), the rotation may pair dimensions 2i and
+2i + 1, and the softmax may have a sink, a learned number per head whose
+exponential is one more term of the denominator. A layer that runs several
+times per token names the cache entry of the pass when it is called.
 """
 
 from __future__ import annotations
@@ -23,7 +28,9 @@ import torch
 import torch.nn as nn
 
 from .. import ops
-from ..parallel.layers import MergedColumnParallelLinear, RowParallelLinear
+from ..parallel.layers import (
+    ColumnParallelLinear, MergedColumnParallelLinear, RowParallelLinear,
+)
 from .forward_meta import ForwardMeta
 from .rope import yarn_ramp_frequencies
 
@@ -33,8 +40,12 @@ class LatentWindowAttention(nn.Module):
                  value_dim: int, rank: int, window: int, scale: float,
                  norm_eps: float, cache_layer_idx: int, owns_cache: bool,
                  rot_dims: Optional[int] = None, rot_base: float = 10000.0,
-                 rot_scaling: Optional[dict] = None):
+                 rot_scaling: Optional[dict] = None, q_rank: int = 0,
+                 rot_interleaved: bool = False, sink: bool = False):
         super().__init__()
+        if q_rank and not owns_cache:
+            raise ValueError("a query latent comes with a cache of its own "
+                             "(both down projections are one GEMM)")
         self.heads, self.dn, self.dr, self.dv = heads, nope_dim, rot_width, value_dim
         self.rank, self.window, self.scale = rank, int(window), float(scale)
         self.eps = norm_eps
@@ -47,44 +58,63 @@ class LatentWindowAttention(nn.Module):
             float(sc.get("original", 0.0)), float(sc.get("fast", 32.0)),
             float(sc.get("slow", 1.0)),
         )
-        sizes = [heads * (nope_dim + rot_width)]
+        self.q_rank, self.rot_interleaved = int(q_rank), bool(rot_interleaved)
+        q_width = heads * (nope_dim + rot_width)
+        sizes = [self.q_rank or q_width]
+        if self.q_rank:
+            self.q_latent_norm = nn.Parameter(torch.empty(self.q_rank),
+                                              requires_grad=False)
+            self.q_up = ColumnParallelLinear(self.q_rank, q_width)
+        self.sink = nn.Parameter(torch.empty(heads), requires_grad=False) \
+            if sink else None
         if owns_cache:
             sizes.append(rank + rot_width)
             self.latent_norm = nn.Parameter(torch.empty(rank), requires_grad=False)
-        # queries (and, for a layer with a cache of its own, the down
-        # projection to latent + rotated key part) in one GEMM
+        # queries or their latent (and, for a layer with a cache of its own,
+        # the down projection to latent + rotated key part) in one GEMM
         self.in_proj = MergedColumnParallelLinear(hidden_size, sizes)
         self.w_uk = nn.Parameter(torch.empty(heads, nope_dim, rank), requires_grad=False)
         self.w_uv = nn.Parameter(torch.empty(heads, value_dim, rank), requires_grad=False)
         self.o_proj = RowParallelLinear(heads * value_dim, hidden_size)
-        self._f32 = None  # (freq, w_uk fp32, w_uv fp32) on the run device
+        self._f32 = None  # (freq, w_uk, w_uv, sink), fp32, on the run device
 
     def _constants(self, device):
         if self._f32 is None or self._f32[0].device != device:
             self._f32 = (self._freq.to(device), self.w_uk.float().contiguous(),
-                         self.w_uv.float().contiguous())
+                         self.w_uv.float().contiguous(),
+                         self.sink.detach().float().contiguous()
+                         if self.sink is not None else None)
         return self._f32
 
     def invalidate_constants(self) -> None:
         self._f32 = None
 
-    def forward(self, x: torch.Tensor, meta: ForwardMeta) -> torch.Tensor:
+    def forward(self, x: torch.Tensor, meta: ForwardMeta,
+                cache_layer_idx: Optional[int] = None) -> torch.Tensor:
         T, H = x.shape[0], self.heads
-        freq, w_uk, w_uv = self._constants(x.device)
+        freq, w_uk, w_uv, sink = self._constants(x.device)
         parts = self.in_proj.split_output(self.in_proj(x))
-        q = parts[0].view(T, H, self.dn + self.dr)
-        cache = meta.mla_cache.layer(self.cache_layer_idx)
+        cache = meta.mla_cache.layer(
+            self.cache_layer_idx if cache_layer_idx is None else cache_layer_idx)
+        q = parts[0]
         if self.owns_cache:
-            ops.latent_kv_store(parts[1], self.latent_norm, self.eps, freq,
-                                self._mult, self.rot_dims, meta.positions,
-                                meta.slot_mapping, cache, self.rank)
+            q_latent = ops.latent_kv_store(
+                parts[1], self.latent_norm, self.eps, freq, self._mult,
+                self.rot_dims, meta.positions, meta.slot_mapping, cache,
+                self.rank, self.rot_interleaved,
+                q if self.q_rank else None,
+                self.q_latent_norm if self.q_rank else None)
+            if self.q_rank:
+                q = self.q_up(q_latent)
+        q = q.view(T, H, self.dn + self.dr)
         q_rot = ops.rope_rows(q, self.dn, self.dr, freq, self._mult,
-                              self.rot_dims, meta.positions)
+                              self.rot_dims, meta.positions,
+                              self.rot_interleaved)
         q_lat = torch.einsum("thd,hdr->thr", q[..., : self.dn].float(), w_uk)
         out_lat = ops.latent_window_attention(
             q_lat.contiguous(), q_rot, cache, meta.block_tables,
             meta.token_seq(), meta.positions, self.window, self.scale,
-            max_seq_len=meta.max_seq_len,
+            max_seq_len=meta.max_seq_len, sink=sink,
         )
         attn = torch.einsum("thr,hvr->thv", out_lat, w_uv).to(x.dtype)
         return self.o_proj(attn.reshape(T, H * self.dv))

@@ -1,5 +1,6 @@
 """Recurrent sequence mixers whose state lives in the engine's per-request
-slots: gated linear attention (below) and minGRU (class MinGRU).
+slots: gated linear attention (below), minGRU (class MinGRU) and the matrix
+LSTM (class MLSTM).
 
 Gated linear attention (GLA): a matrix-valued recurrent state per head with
 a data-dependent decay per key channel,
@@ -113,3 +114,65 @@ class MinGRU(nn.Module):
 
     def forward(self, x: torch.Tensor, meta: ForwardMeta) -> torch.Tensor:
         return self.o_proj(self.mix(self.in_proj(x), meta))
+
+
+class MLSTM(nn.Module):
+    """Matrix LSTM (the mLSTM cell of xLSTM): per head a matrix memory S
+    [dim, vdim], a normaliser n [dim] and a running maximum m with scalar
+    exponential gates,
+
+        i = cap tanh((W_i h + b_i) / cap),
+        f = logsigmoid(cap tanh((W_f h + b_f) / cap)),
+        m' = max(f + m, i),
+        S <- exp(f + m - m') S + exp(i - m') k v^T,   n likewise with k alone,
+        o = S^T q / (max(|n . q|, exp(-m')) + 1e-6),   q = W_q h / sqrt(dim),
+
+    all three starting at zero; each head's o is divided by its RMS, the heads
+    together are multiplied by a weight and by sigmoid(W_g h) before the
+    output projection. State, gates, normalisation and output gate are fp32
+    (ops.mlstm); so are the gates' pre-activations (ops.linear_f32), which end
+    in exponentials. The state lives in LinearStateCache slots, one row
+    [S | n | m] per head. A layer that runs several times per token names the
+    state of the pass when it is called."""
+
+    def __init__(self, hidden_size: int, heads: int, dim: int, vdim: int,
+                 gate_cap: float, norm_eps: float, state_layer_idx: int = 0):
+        super().__init__()
+        self.heads, self.dim, self.vdim = heads, dim, vdim
+        self.cap, self.eps = float(gate_cap), float(norm_eps)
+        self.state_layer_idx = state_layer_idx
+        # one GEMM for q | k | v | output gate
+        self.in_proj = MergedColumnParallelLinear(
+            hidden_size, [heads * dim, heads * dim, heads * vdim, heads * vdim])
+        # input gates, then forget gates
+        self.gate_weight = nn.Parameter(torch.empty(2 * heads, hidden_size),
+                                        requires_grad=False)
+        self.gate_bias = nn.Parameter(torch.empty(2 * heads), requires_grad=False)
+        self.norm_weight = nn.Parameter(torch.empty(heads * vdim),
+                                        requires_grad=False)
+        self.o_proj = RowParallelLinear(heads * vdim, hidden_size)
+        self._b32 = None
+
+    def load_gate(self, which: int, w=None, b=None) -> None:
+        """which: 0 = input gate, 1 = forget gate."""
+        rows = slice(which * self.heads, (which + 1) * self.heads)
+        if w is not None:
+            self.gate_weight.data[rows].copy_(w)
+        if b is not None:
+            self.gate_bias.data[rows].copy_(b)
+
+    def invalidate_constants(self) -> None:
+        self._b32 = None
+
+    def forward(self, x: torch.Tensor, meta: ForwardMeta,
+                state_layer_idx=None) -> torch.Tensor:
+        if self._b32 is None or self._b32.device != x.device:
+            self._b32 = self.gate_bias.detach().float().contiguous()
+        q, k, v, g = self.in_proj.split_output(self.in_proj(x))
+        idx = self.state_layer_idx if state_layer_idx is None else state_layer_idx
+        o = ops.mlstm(q, k, v, g, ops.linear_f32(x, self.gate_weight),
+                      self._b32, self.norm_weight, self.cap, self.eps,
+                      meta.linear_cache.recurrent_states[idx],
+                      meta.linear_slots, meta.query_bounds(), meta.positions,
+                      x.dtype)
+        return self.o_proj(o)

@@ -17,15 +17,27 @@ import torch.nn.functional as F
 
 from .. import ops
 from ..parallel.comm import get_comm
+from ..parallel.layers import MergedColumnParallelLinear, RowParallelLinear
 from .config import ModelConfig
 
 
 class MoERouter(nn.Module):
     """Top-k router. Supports softmax scoring (Qwen/GLM style) and sigmoid
-    scoring with bias correction + group-limited top-k (DeepSeek-V3 style)."""
+    scoring with bias correction + group-limited top-k (DeepSeek-V3 style).
 
-    def __init__(self, cfg: ModelConfig):
+    logit_bias: softmax scoring adds a learned number per expert to its logit
+    (before the choice). extra_rows: further rows of the same weight that are
+    no experts (a shared expert's gate, say); route() returns their fp32
+    outputs beside the routing. Both want softmax scoring with weights
+    normalised over the chosen experts and run in one kernel (ops.route_softmax)."""
+
+    def __init__(self, cfg: ModelConfig, logit_bias: bool = False,
+                 extra_rows: int = 0):
         super().__init__()
+        self.fused = logit_bias or extra_rows > 0
+        if self.fused and (cfg.scoring_func != "softmax" or not cfg.norm_topk_prob):
+            raise ValueError("logit bias and extra rows come with softmax "
+                             "weights over the chosen experts")
         self.num_experts = cfg.num_experts
         self.top_k = cfg.num_experts_per_tok
         self.norm_topk_prob = cfg.norm_topk_prob
@@ -34,16 +46,34 @@ class MoERouter(nn.Module):
         self.n_group = cfg.n_group
         self.topk_group = cfg.topk_group
         self.weight = nn.Parameter(
-            torch.empty(cfg.num_experts, cfg.hidden_size), requires_grad=False
+            torch.empty(cfg.num_experts + extra_rows, cfg.hidden_size),
+            requires_grad=False
         )
+        self.logit_bias = nn.Parameter(
+            torch.zeros(cfg.num_experts), requires_grad=False
+        ) if logit_bias else None
+        self._b32 = None
         if cfg.scoring_func == "sigmoid":
             # DeepSeek-V3 e_score_correction_bias
             self.e_score_correction_bias = nn.Parameter(
                 torch.zeros(cfg.num_experts), requires_grad=False
             )
 
+    def invalidate_constants(self) -> None:
+        self._b32 = None
+
+    def route(self, x: torch.Tensor):
+        """x: [T, H] -> (ids [T, k], weights [T, k], extra rows' outputs)."""
+        if self.logit_bias is not None and (
+                self._b32 is None or self._b32.device != x.device):
+            self._b32 = self.logit_bias.detach().float().contiguous()
+        return ops.route_softmax(x, self.weight, self._b32, self.num_experts,
+                                 self.top_k)
+
     def forward(self, x: torch.Tensor):
         """x: [T, H] -> (topk_ids [T, k] long, topk_weights [T, k] float)."""
+        if self.fused:
+            return self.route(x)[:2]
         logits = F.linear(x.float(), self.weight.float())
         if self.scoring_func == "sigmoid":
             scores = logits.sigmoid()
@@ -86,7 +116,7 @@ class FusedMoE(nn.Module):
     replication."""
 
     def __init__(self, cfg: ModelConfig, intermediate_size: Optional[int] = None,
-                 act_limit: float = 0.0):
+                 act_limit: float = 0.0, router: Optional[MoERouter] = None):
         super().__init__()
         self.cfg = cfg
         # act_limit > 0: gpt-oss/minimax-m3 clamped swiglu
@@ -102,7 +132,7 @@ class FusedMoE(nn.Module):
         self.ep_rank = comm.tp_rank if self.ep_size > 1 else 0
         self.num_local_experts = E // self.ep_size
         self.expert_offset = self.ep_rank * self.num_local_experts
-        self.router = MoERouter(cfg)
+        self.router = router if router is not None else MoERouter(cfg)
         self.fp8 = False
         self.w_gate_up = nn.Parameter(
             torch.empty(self.num_local_experts, 2 * inter, H), requires_grad=False
@@ -204,9 +234,11 @@ class FusedMoE(nn.Module):
         o = self.expert_offset
         self.w_down.data.copy_(t[o : o + self.num_local_experts])
 
-    def forward(self, x: torch.Tensor) -> torch.Tensor:
+    def forward(self, x: torch.Tensor, routing=None) -> torch.Tensor:
+        """routing: (ids, weights) from a caller that has run the router."""
         T, H = x.shape
-        topk_ids, topk_w = self.router(x)           # [T,k] global expert ids
+        # [T,k] global expert ids
+        topk_ids, topk_w = routing if routing is not None else self.router(x)
         if self.routing_counts is not None:
             self.routing_counts.scatter_add_(
                 0, topk_ids.reshape(-1),
@@ -303,3 +335,35 @@ class MoEBlock(nn.Module):
         if self.shared is not None:
             y = y + self.shared(x)
         return y
+
+
+class SharedExpertMoE(nn.Module):
+    """Routed experts (softmax over the chosen logits, a logit bias per
+    expert) plus a shared expert whose result is multiplied by sigmoid(w . x),
+    one number per token. The gate's row rides in the router's weight.
+    forward returns the parts (routed sum, fp32; shared result; gate
+    pre-activation [T] fp32; the last two None without a shared expert) so
+    that the caller's residual kernel gates and adds in fp32."""
+
+    def __init__(self, cfg: ModelConfig, shared_ff: int = 0):
+        super().__init__()
+        self.experts = FusedMoE(cfg, router=MoERouter(
+            cfg, logit_bias=True, extra_rows=1 if shared_ff else 0))
+        self.experts.fp32_output = True
+        self.shared_ff = int(shared_ff)
+        self.gate_up = self.down = None
+        if shared_ff:
+            self.gate_up = MergedColumnParallelLinear(
+                cfg.hidden_size, [shared_ff, shared_ff])
+            self.down = RowParallelLinear(shared_ff, cfg.hidden_size)
+
+    def invalidate_constants(self) -> None:
+        self.experts.router.invalidate_constants()
+
+    def forward(self, x: torch.Tensor):
+        ids, wts, rest = self.experts.router.route(x)
+        y = self.experts(x, routing=(ids, wts))
+        if not self.shared_ff:
+            return y, None, None
+        s = self.down(ops.biased_glu(self.gate_up(x), None, "silu"))
+        return y, s, rest

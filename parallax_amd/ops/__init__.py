@@ -649,22 +649,29 @@ apply_penalties = ref.apply_penalties
 # -- sequence mixers (extension _mix) ------------------------------------------
 from .mix import (  # noqa: E402,F401
     add_layernorm,
+    biased_glu,
     branch_rmsnorm_add,
     clamped_glu,
+    embed_streams,
     gated_rmsnorm,
     gla_recurrence,
     group_rmsnorm_add,
     has_mix_extension,
+    hyper_rmsnorm,
     latent_kv_store,
     latent_window_attention,
+    linear_f32,
     mingru_scan,
+    mlstm,
     pair_hash_embedding,
     pool_cache_update,
     qkv_store,
     relu_squared,
     rope_rows,
     rotate_heads,
+    route_softmax,
     row_attention,
     sandwich_rmsnorm,
+    softcap_logits,
     xielu,
 )

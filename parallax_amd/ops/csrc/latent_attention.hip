@@ -9,7 +9,8 @@
 // activation type.
 //
 //   latent_kv_store : RMS norm of the latent + rotation of the key part +
-//                     scatter into the paged cache, one kernel per layer.
+//                     scatter into the paged cache, one kernel per layer (and,
+//                     where queries come through a latent, its RMS norm too).
 //   rope_rows       : rotation of the queries' rotated part into an fp32 buffer.
 //   latent_window_attention : a workgroup per (token, group of heads, share of
 //                     the keys); 64 keys per wave and pass, online softmax,
@@ -21,17 +22,39 @@
 //                     small kernel joins the partial results.
 //
 // Angles are computed in fp32 from a per-layer frequency vector: pair
-// (i, i + rot_dims/2), a = pos * freq[i], cos and sin scaled by `mult`.
+// (i, i + rot_dims/2), or (2i, 2i + 1) with `inter`, a = pos * freq[i], cos and
+// sin scaled by `mult`. A sink (one number per head) is one more term of the
+// softmax's denominator, exp(sink), without a value: the running maximum of
+// one wave starts at it with the denominator 1.
 #include "seq_common.h"
 
+// grid (tokens, 1 or 2): blockIdx.y 1 norms the token's query latent
 template <typename T>
 __global__ __launch_bounds__(128) void latent_kv_store_kernel(
     const T* __restrict__ dkv, int64_t dkv_stride, const T* __restrict__ norm_w,
     float eps, const float* __restrict__ freq, float mult, int rot_dims,
-    const int* __restrict__ positions, const int64_t* __restrict__ slots,
-    T* __restrict__ cache, int rank, int rot_w) {
+    int inter, const int* __restrict__ positions,
+    const int64_t* __restrict__ slots, T* __restrict__ cache, int rank,
+    int rot_w, T* __restrict__ q_out, const T* __restrict__ q_down,
+    int64_t q_stride, const T* __restrict__ q_norm_w, int q_rank) {
   __shared__ float scratch[4];
   const int64_t t = blockIdx.x;
+  if (blockIdx.y == 1) {
+    const T* x = q_down + t * q_stride;
+    float sq = 0.f;
+    for (int i = threadIdx.x; i < q_rank; i += 128) {
+      const float v = ldf(x + i);
+      sq += v * v;
+    }
+    sq = wave_reduce_sum(sq);
+    if ((threadIdx.x & 63) == 0) scratch[threadIdx.x >> 6] = sq;
+    __syncthreads();
+    const float r = 1.0f / sqrtf((scratch[0] + scratch[1]) / (float)q_rank + eps);
+    T* o = q_out + t * (int64_t)q_rank;
+    for (int i = threadIdx.x; i < q_rank; i += 128)
+      stf(o + i, ldf(x + i) * r * ldf(q_norm_w + i));
+    return;
+  }
   const int64_t slot = slots[t];
   if (slot < 0) return;  // pad row of a captured graph
   const T* x = dkv + t * dkv_stride;
@@ -58,9 +81,10 @@ __global__ __launch_bounds__(128) void latent_kv_store_kernel(
     sincosf(p * freq[i], &s, &c);
     s *= mult;
     c *= mult;
-    const float u = ldf(kx + i), v = ldf(kx + i + half);
-    stf(kd + i, u * c - v * s);
-    stf(kd + i + half, v * c + u * s);
+    const int iu = inter ? 2 * i : i, iv = inter ? 2 * i + 1 : i + half;
+    const float u = ldf(kx + iu), v = ldf(kx + iv);
+    stf(kd + iu, u * c - v * s);
+    stf(kd + iv, v * c + u * s);
   }
   for (int i = rot_dims + threadIdx.x; i < rot_w; i += 128) {
     stf(kd + i, ldf(kx + i));
@@ -73,7 +97,8 @@ template <typename T>
 __global__ __launch_bounds__(256) void rope_rows_kernel(
     float* __restrict__ out, const T* __restrict__ q, int64_t tok_stride,
     int64_t head_stride, int col0, const float* __restrict__ freq, float mult,
-    int rot_dims, const int* __restrict__ positions, int H, int rot_w) {
+    int rot_dims, int inter, const int* __restrict__ positions, int H,
+    int rot_w) {
   extern __shared__ float cs[];  // [rot_dims/2] cos, [rot_dims/2] sin
   const int64_t t = blockIdx.x;
   const int half = rot_dims >> 1;
@@ -91,9 +116,10 @@ __global__ __launch_bounds__(256) void rope_rows_kernel(
     const T* src = q + t * tok_stride + h * head_stride + col0;
     float* dst = out + (t * H + h) * (int64_t)rot_w;
     if (i < half) {
-      const float u = ldf(src + i), v = ldf(src + i + half);
-      dst[i] = u * cs[i] - v * cs[half + i];
-      dst[i + half] = v * cs[i] + u * cs[half + i];
+      const int iu = inter ? 2 * i : i, iv = inter ? 2 * i + 1 : i + half;
+      const float u = ldf(src + iu), v = ldf(src + iv);
+      dst[iu] = u * cs[i] - v * cs[half + i];
+      dst[iv] = v * cs[i] + u * cs[half + i];
     } else {
       const int k = rot_dims + (i - half);
       dst[k] = ldf(src + k);
@@ -137,7 +163,8 @@ __global__ __launch_bounds__(256) void latent_window_attention_kernel(
     const T* __restrict__ cache, const int* __restrict__ block_tables,
     int bt_stride, const int* __restrict__ token_seq,
     const int* __restrict__ positions, int H, int rank, int rot_w,
-    int block_size, int window, float scale, int splits) {
+    int block_size, int window, float scale, int splits,
+    const float* __restrict__ sink) {
   extern __shared__ float lds[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int64_t t = blockIdx.x;
@@ -167,8 +194,10 @@ __global__ __launch_bounds__(256) void latent_window_attention_kernel(
   float m[HB], l[HB], acc[HB][RC][8];
 #pragma unroll
   for (int h = 0; h < HB; ++h) {
-    m[h] = -INFINITY;
-    l[h] = 0.f;
+    // the sink is counted once: by the first wave of the first share
+    const bool here = sink != nullptr && split == 0 && wave == 0;
+    m[h] = here ? sink[min(h0 + h, H - 1)] : -INFINITY;
+    l[h] = here ? 1.f : 0.f;
 #pragma unroll
     for (int c = 0; c < RC; ++c)
 #pragma unroll
@@ -353,38 +382,41 @@ __global__ __launch_bounds__(256) void latent_window_reduce_kernel(
 extern "C" void launch_latent_kv_store(const void* dkv, int64_t dkv_stride,
                                        const void* norm_w, float eps,
                                        const float* freq, float mult,
-                                       int rot_dims, const int* positions,
+                                       int rot_dims, int inter,
+                                       const int* positions,
                                        const int64_t* slots, void* cache,
-                                       int rank, int rot_w, int T, int kind,
-                                       hipStream_t stream) {
+                                       int rank, int rot_w, void* q_out,
+                                       const void* q_down, int64_t q_stride,
+                                       const void* q_norm_w, int q_rank, int T,
+                                       int kind, hipStream_t stream) {
   if (T == 0) return;
-  if (kind == 0)
-    hipLaunchKernelGGL((latent_kv_store_kernel<bf16_t>), dim3(T), dim3(128), 0,
-                       stream, (const bf16_t*)dkv, dkv_stride,
-                       (const bf16_t*)norm_w, eps, freq, mult, rot_dims,
-                       positions, slots, (bf16_t*)cache, rank, rot_w);
-  else
-    hipLaunchKernelGGL((latent_kv_store_kernel<float>), dim3(T), dim3(128), 0,
-                       stream, (const float*)dkv, dkv_stride,
-                       (const float*)norm_w, eps, freq, mult, rot_dims,
-                       positions, slots, (float*)cache, rank, rot_w);
+#define LK_CALL(TT)                                                            \
+  hipLaunchKernelGGL((latent_kv_store_kernel<TT>), dim3(T, q_rank > 0 ? 2 : 1), \
+                     dim3(128), 0, stream, (const TT*)dkv, dkv_stride,         \
+                     (const TT*)norm_w, eps, freq, mult, rot_dims, inter,      \
+                     positions, slots, (TT*)cache, rank, rot_w, (TT*)q_out,    \
+                     (const TT*)q_down, q_stride, (const TT*)q_norm_w, q_rank)
+  if (kind == 0) LK_CALL(bf16_t);
+  else LK_CALL(float);
+#undef LK_CALL
 }
 
 extern "C" void launch_rope_rows(float* out, const void* q, int64_t tok_stride,
                                  int64_t head_stride, int col0,
                                  const float* freq, float mult, int rot_dims,
-                                 const int* positions, int H, int rot_w, int T,
-                                 int kind, hipStream_t stream) {
+                                 int inter, const int* positions, int H,
+                                 int rot_w, int T, int kind,
+                                 hipStream_t stream) {
   if (T == 0) return;
   const size_t shm = sizeof(float) * (size_t)rot_dims;
   if (kind == 0)
     hipLaunchKernelGGL((rope_rows_kernel<bf16_t>), dim3(T), dim3(256), shm,
                        stream, out, (const bf16_t*)q, tok_stride, head_stride,
-                       col0, freq, mult, rot_dims, positions, H, rot_w);
+                       col0, freq, mult, rot_dims, inter, positions, H, rot_w);
   else
     hipLaunchKernelGGL((rope_rows_kernel<float>), dim3(T), dim3(256), shm,
                        stream, out, (const float*)q, tok_stride, head_stride,
-                       col0, freq, mult, rot_dims, positions, H, rot_w);
+                       col0, freq, mult, rot_dims, inter, positions, H, rot_w);
 }
 
 template <typename T, int HB, int RC>
@@ -393,7 +425,8 @@ static void launch_lwa_hb(float* out, float* part, const float* q_lat,
                           const int* block_tables, int bt_stride,
                           const int* token_seq, const int* positions, int T_,
                           int H, int rank, int rot_w, int block_size, int window,
-                          float scale, int splits, hipStream_t stream) {
+                          float scale, int splits, const float* sink,
+                          hipStream_t stream) {
   const int E = rank + rot_w;
   const int Ep = (E + 7) & ~7;
   const int rank8 = (rank + 7) & ~7;
@@ -407,13 +440,13 @@ static void launch_lwa_hb(float* out, float* part, const float* q_lat,
                        dim3(256), shm, stream, out, part, q_lat, q_rot,
                        (const T*)cache, block_tables, bt_stride, token_seq,
                        positions, H, rank, rot_w, block_size, window, scale,
-                       splits);
+                       splits, sink);
   else
     hipLaunchKernelGGL((latent_window_attention_kernel<T, HB, RC, false>), grid,
                        dim3(256), shm, stream, out, part, q_lat, q_rot,
                        (const T*)cache, block_tables, bt_stride, token_seq,
                        positions, H, rank, rot_w, block_size, window, scale,
-                       splits);
+                       splits, sink);
   if (splits > 1)
     hipLaunchKernelGGL(latent_window_reduce_kernel, dim3(T_ * H), dim3(256), 0,
                        stream, out, part, rank, splits);
@@ -425,10 +458,11 @@ static void launch_lwa_t(float* out, float* part, const float* q_lat,
                          const int* block_tables, int bt_stride,
                          const int* token_seq, const int* positions, int T_,
                          int H, int rank, int rot_w, int block_size, int window,
-                         float scale, int splits, hipStream_t stream) {
+                         float scale, int splits, const float* sink,
+                          hipStream_t stream) {
 #define LWA_ARGS                                                             \
   out, part, q_lat, q_rot, cache, block_tables, bt_stride, token_seq,         \
-      positions, T_, H, rank, rot_w, block_size, window, scale, splits, stream
+      positions, T_, H, rank, rot_w, block_size, window, scale, splits, sink, stream
   // heads per workgroup: 8 where the latent accumulators fit the registers
   // (rank <= 512), 4 above; fewer when the model has fewer heads
   if (rank <= 512) {
@@ -448,15 +482,15 @@ extern "C" void launch_latent_window_attention(
     float* out, float* part, const float* q_lat, const float* q_rot,
     const void* cache, const int* block_tables, int bt_stride,
     const int* token_seq, const int* positions, int T, int H, int rank,
-    int rot_w, int block_size, int window, float scale, int splits, int kind,
-    hipStream_t stream) {
+    int rot_w, int block_size, int window, float scale, int splits,
+    const float* sink, int kind, hipStream_t stream) {
   if (T == 0) return;
   if (kind == 0)
     launch_lwa_t<bf16_t>(out, part, q_lat, q_rot, cache, block_tables,
                          bt_stride, token_seq, positions, T, H, rank, rot_w,
-                         block_size, window, scale, splits, stream);
+                         block_size, window, scale, splits, sink, stream);
   else
     launch_lwa_t<float>(out, part, q_lat, q_rot, cache, block_tables, bt_stride,
                         token_seq, positions, T, H, rank, rot_w, block_size,
-                        window, scale, splits, stream);
+                        window, scale, splits, sink, stream);
 }

@@ -1,7 +1,8 @@
 // Python bindings of the sequence-mixer kernels (extension parallax_amd.ops._mix):
 // fp32-residual layer norm, sliding-window latent attention, gated linear
 // attention, sandwich RMS norm with depth averaging, row-cache attention
-// (differential / pooled sliding window), xIELU. Every entry point checks shapes and types on the host before a
+// (differential / pooled sliding window), xIELU, hyper-connected streams,
+// matrix LSTM, softmax router. Every entry point checks shapes and types on the host before a
 // launch; activation tensors are bf16 or float32 (one template instance each).
 
 #include <ATen/hip/HIPContext.h>
@@ -10,21 +11,43 @@
 #include <hip/hip_runtime.h>
 
 #include <algorithm>
+#include <cmath>
 
 extern "C" {
 void launch_add_layernorm(float*, const void*, int64_t, int, const void*, float,
                           const void*, const void*, float, void*, int, int, int,
                           hipStream_t);
 void launch_latent_kv_store(const void*, int64_t, const void*, float,
-                            const float*, float, int, const int*,
-                            const int64_t*, void*, int, int, int, int,
+                            const float*, float, int, int, const int*,
+                            const int64_t*, void*, int, int, void*,
+                            const void*, int64_t, const void*, int, int, int,
                             hipStream_t);
 void launch_rope_rows(float*, const void*, int64_t, int64_t, int, const float*,
-                      float, int, const int*, int, int, int, int, hipStream_t);
+                      float, int, int, const int*, int, int, int, int,
+                      hipStream_t);
 void launch_latent_window_attention(float*, float*, const float*, const float*,
                                     const void*, const int*, int, const int*,
                                     const int*, int, int, int, int, int, int,
-                                    float, int, int, hipStream_t);
+                                    float, int, const float*, int, hipStream_t);
+void launch_hyper_rmsnorm(float*, const void*, int, int64_t, const void*,
+                          const void*, int64_t, const float*, int64_t,
+                          const float*, const float*, const float*, const void*,
+                          float, void*, int, int, int, int, hipStream_t);
+void launch_embed_streams(float*, const int64_t*, const void*, int64_t, int,
+                          int, int, int, hipStream_t);
+void launch_biased_glu(void*, const void*, int64_t, const void*, int, int, int,
+                       int, hipStream_t);
+void launch_softcap_logits(float*, const void*, float, float, int64_t, int,
+                           hipStream_t);
+void launch_small_linear(float*, const void*, int64_t, const void*, int, int,
+                         int, int64_t*, float*, const float*, int, int,
+                         hipStream_t);
+void launch_mlstm(void*, float*, float*, float*, const void*, int64_t,
+                  const void*, int64_t, const void*, int64_t, const void*,
+                  int64_t, const float*, const float*, const void*, float,
+                  float, float*, int64_t, const int64_t*, const int*,
+                  const int*, int, int, int, int, int, float, int, int,
+                  hipStream_t);
 void launch_gla_recurrence(float*, const void*, const void*, const void*,
                            const void*, int64_t, int64_t, int64_t, int64_t,
                            const void*, float*, const int64_t*, const int*,
@@ -150,8 +173,20 @@ void add_layernorm(torch::Tensor resid, torch::Tensor y, torch::Tensor scale,
 void latent_kv_store(torch::Tensor dkv, torch::Tensor norm_w, double eps,
                      torch::Tensor freq, double mult, int64_t rot_dims,
                      torch::Tensor positions, torch::Tensor slots,
-                     torch::Tensor cache, int64_t rank) {
+                     torch::Tensor cache, int64_t rank, bool interleaved,
+                     torch::Tensor q_down, torch::Tensor q_norm_w,
+                     torch::Tensor q_out) {
   const int kind = kind_of(dkv, "dkv");
+  // q_down [T, q_rank] (row stride free) or empty: also normed, into q_out
+  const bool has_q = q_down.numel() > 0 && q_down.dim() == 2;
+  if (has_q) {
+    TORCH_CHECK(q_down.is_cuda() && q_down.scalar_type() == dkv.scalar_type() &&
+                q_down.size(0) == dkv.size(0) && q_down.stride(1) == 1);
+    TORCH_CHECK(q_norm_w.is_cuda() && q_norm_w.scalar_type() == dkv.scalar_type() &&
+                q_norm_w.is_contiguous() && q_norm_w.numel() == q_down.size(1));
+    TORCH_CHECK(q_out.is_cuda() && q_out.scalar_type() == dkv.scalar_type() &&
+                q_out.is_contiguous() && q_out.sizes() == q_down.sizes());
+  }
   TORCH_CHECK(dkv.dim() == 2 && dkv.stride(1) == 1);
   const int T = dkv.size(0);
   const int rot_w = dkv.size(1) - rank;
@@ -168,16 +203,21 @@ void latent_kv_store(torch::Tensor dkv, torch::Tensor norm_w, double eps,
   TORCH_CHECK(positions.numel() == T && slots.numel() == T);
   launch_latent_kv_store(dkv.data_ptr(), dkv.stride(0), norm_w.data_ptr(),
                          (float)eps, freq.data_ptr<float>(), (float)mult,
-                         (int)rot_dims, positions.data_ptr<int>(),
-                         slots.data_ptr<int64_t>(), cache.data_ptr(), (int)rank,
-                         rot_w, T, kind, cur_stream());
+                         (int)rot_dims, interleaved ? 1 : 0,
+                         positions.data_ptr<int>(), slots.data_ptr<int64_t>(),
+                         cache.data_ptr(), (int)rank, rot_w,
+                         has_q ? q_out.data_ptr() : nullptr,
+                         has_q ? q_down.data_ptr() : nullptr,
+                         has_q ? q_down.stride(0) : 0,
+                         has_q ? q_norm_w.data_ptr() : nullptr,
+                         has_q ? (int)q_down.size(1) : 0, T, kind, cur_stream());
 }
 
 // q [T, H, D] (strided view); rotates columns [col0, col0 + rot_w) of every
 // head into out [T, H, rot_w] fp32
 void rope_rows(torch::Tensor out, torch::Tensor q, int64_t col0,
                torch::Tensor freq, double mult, int64_t rot_dims,
-               torch::Tensor positions) {
+               torch::Tensor positions, bool interleaved) {
   const int kind = kind_of(q, "q");
   CHECK_F32C(out);
   TORCH_CHECK(q.dim() == 3 && out.dim() == 3 && q.stride(2) == 1);
@@ -191,8 +231,8 @@ void rope_rows(torch::Tensor out, torch::Tensor q, int64_t col0,
   TORCH_CHECK(positions.numel() == T);
   launch_rope_rows(out.data_ptr<float>(), q.data_ptr(), q.stride(0),
                    q.stride(1), (int)col0, freq.data_ptr<float>(), (float)mult,
-                   (int)rot_dims, positions.data_ptr<int>(), H, rot_w, T, kind,
-                   cur_stream());
+                   (int)rot_dims, interleaved ? 1 : 0,
+                   positions.data_ptr<int>(), H, rot_w, T, kind, cur_stream());
 }
 
 // out/q_lat [T, H, rank] fp32, q_rot [T, H, rot_w] fp32, cache [blocks, block,
@@ -202,8 +242,14 @@ void latent_window_attention(torch::Tensor out, torch::Tensor q_lat,
                              torch::Tensor q_rot, torch::Tensor cache,
                              torch::Tensor block_tables, torch::Tensor token_seq,
                              torch::Tensor positions, int64_t window,
-                             double scale, int64_t max_keys) {
+                             double scale, int64_t max_keys,
+                             torch::Tensor sink) {
   const int kind = kind_of(cache, "cache");
+  const bool has_sink = sink.numel() > 0;   // [H] fp32
+  if (has_sink) {
+    CHECK_F32C(sink);
+    TORCH_CHECK(q_lat.dim() == 3 && sink.numel() == q_lat.size(1), "sinks");
+  }
   CHECK_F32C(out);
   CHECK_F32C(q_lat);
   CHECK_F32C(q_rot);
@@ -248,7 +294,7 @@ void latent_window_attention(torch::Tensor out, torch::Tensor q_lat,
       block_tables.data_ptr<int>(), (int)block_tables.stride(0),
       has_seq ? token_seq.data_ptr<int>() : nullptr, positions.data_ptr<int>(),
       T, H, rank, rot_w, (int)cache.size(1), (int)window, (float)scale, splits,
-      kind, cur_stream());
+      has_sink ? sink.data_ptr<float>() : nullptr, kind, cur_stream());
 }
 
 // q, k, z [T, H*dk] and v [T, H*dv] (row strides free), z_bias [H*dk],
@@ -839,6 +885,213 @@ void mingru_scan(torch::Tensor out, torch::Tensor zug, torch::Tensor z_bias,
                      positions.data_ptr<int>(), B, width, kind, cur_stream());
 }
 
+// x [T, S * W] fp32 in place; y [T, W] (activation type or fp32, row stride
+// free) or empty = no update; y_bias [W], y2 [T, W] + gate2 [T] fp32 or empty;
+// mix [S, S], wr [S] fp32; rd [S] fp32 + weight [W] + out [T, W] or empty
+void hyper_rmsnorm(torch::Tensor x, torch::Tensor y, torch::Tensor y_bias,
+                   torch::Tensor y2, torch::Tensor gate2, torch::Tensor mix,
+                   torch::Tensor wr, torch::Tensor rd, torch::Tensor weight,
+                   double eps, torch::Tensor out, int64_t S) {
+  CHECK_F32C(x);
+  TORCH_CHECK(x.dim() == 2 && S >= 1 && x.size(1) % S == 0);
+  TORCH_CHECK(S <= 16, "more than 16 residual streams are not supported");
+  const int rows = x.size(0), W = x.size(1) / S;
+  const bool has_y = y.numel() > 0, has_r = rd.numel() > 0;
+  const bool has_b = has_y && y_bias.numel() > 0, has_y2 = has_y && y2.numel() > 0;
+  TORCH_CHECK(has_y || has_r || rows == 0, "nothing to do");
+  int kind = kind_of(out, "out");   // the activation type, also when empty
+  bool y_f32 = false;
+  if (has_y) {
+    y_f32 = y.scalar_type() == at::kFloat && kind == 0;
+    TORCH_CHECK(y.is_cuda() && y.dim() == 2 && y.size(0) == rows &&
+                y.size(1) == W && y.stride(1) == 1 &&
+                (y_f32 || y.scalar_type() == out.scalar_type()), "y");
+    CHECK_F32C(mix);
+    CHECK_F32C(wr);
+    TORCH_CHECK(mix.numel() == S * S && wr.numel() == S, "stream coefficients");
+  }
+  if (has_b)
+    TORCH_CHECK(y_bias.is_cuda() && y_bias.scalar_type() == out.scalar_type() &&
+                y_bias.is_contiguous() && y_bias.numel() == W, "y_bias");
+  if (has_y2) {
+    TORCH_CHECK(y2.is_cuda() && y2.scalar_type() == out.scalar_type() &&
+                y2.dim() == 2 && y2.size(0) == rows && y2.size(1) == W &&
+                y2.stride(1) == 1, "y2");
+    CHECK_F32C(gate2);
+    TORCH_CHECK(gate2.numel() == rows, "gate2");
+  }
+  if (has_r) {
+    CHECK_F32C(rd);
+    TORCH_CHECK(rd.numel() == S, "stream coefficients");
+    TORCH_CHECK(weight.is_cuda() && weight.scalar_type() == out.scalar_type() &&
+                weight.is_contiguous() && weight.numel() == W, "weight");
+    TORCH_CHECK(out.is_contiguous() && out.dim() == 2 && out.size(0) == rows &&
+                out.size(1) == W, "out");
+  }
+  launch_hyper_rmsnorm(
+      x.data_ptr<float>(), has_y ? y.data_ptr() : nullptr, y_f32 ? 1 : 0,
+      has_y ? y.stride(0) : 0, has_b ? y_bias.data_ptr() : nullptr,
+      has_y2 ? y2.data_ptr() : nullptr, has_y2 ? y2.stride(0) : 0,
+      has_y2 ? gate2.data_ptr<float>() : nullptr, 1,
+      has_y ? mix.data_ptr<float>() : nullptr,
+      has_y ? wr.data_ptr<float>() : nullptr,
+      has_r ? rd.data_ptr<float>() : nullptr,
+      has_r ? weight.data_ptr() : nullptr, (float)eps,
+      has_r ? out.data_ptr() : nullptr, rows, W, (int)S, kind, cur_stream());
+}
+
+// out [T, S * W] fp32, ids [T] int64, table [V, W]
+void embed_streams(torch::Tensor out, torch::Tensor ids, torch::Tensor table,
+                   int64_t S) {
+  const int kind = kind_of(table, "table");
+  CHECK_F32C(out);
+  CHECK_I64(ids);
+  TORCH_CHECK(table.dim() == 2 && table.is_contiguous() && S >= 1 &&
+              out.dim() == 2 && out.size(0) == ids.numel() &&
+              out.size(1) == S * table.size(1));
+  launch_embed_streams(out.data_ptr<float>(), ids.data_ptr<int64_t>(),
+                       table.data_ptr(), table.size(0), (int)table.size(1),
+                       (int)S, (int)ids.numel(), kind, cur_stream());
+}
+
+// x [rows, 2 I] (row stride free), bias [2 I] or empty -> out [rows, I]
+void biased_glu(torch::Tensor out, torch::Tensor x, torch::Tensor bias, bool gelu) {
+  const int kind = kind_of(x, "x");
+  TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1 && x.size(1) % 2 == 0);
+  const int rows = x.size(0), I = x.size(1) / 2;
+  TORCH_CHECK(out.is_cuda() && out.scalar_type() == x.scalar_type() &&
+              out.is_contiguous() && out.dim() == 2 && out.size(0) == rows &&
+              out.size(1) == I);
+  const bool has_b = bias.numel() > 0;
+  if (has_b)
+    TORCH_CHECK(bias.is_cuda() && bias.scalar_type() == x.scalar_type() &&
+                bias.is_contiguous() && bias.numel() == 2 * I);
+  launch_biased_glu(out.data_ptr(), x.data_ptr(), x.stride(0),
+                    has_b ? bias.data_ptr() : nullptr, I, rows, gelu ? 1 : 0,
+                    kind, cur_stream());
+}
+
+void softcap_logits(torch::Tensor out, torch::Tensor x, double scale, double cap) {
+  const int kind = kind_of(x, "x");
+  CHECK_F32C(out);
+  TORCH_CHECK(x.is_contiguous() && out.numel() == x.numel());
+  launch_softcap_logits(out.data_ptr<float>(), x.data_ptr(), (float)scale,
+                        (float)cap, x.numel(), kind, cur_stream());
+}
+
+static void check_small_linear(const torch::Tensor& x, const torch::Tensor& w) {
+  TORCH_CHECK(x.is_cuda() && x.scalar_type() == at::kBFloat16 && x.dim() == 2 &&
+              x.stride(1) == 1, "x must be bf16 rows");
+  TORCH_CHECK(w.is_cuda() && w.scalar_type() == at::kBFloat16 && w.dim() == 2 &&
+              w.is_contiguous() && w.size(1) == x.size(1), "weight");
+}
+
+// out [T, N] fp32 = x [T, K] bf16 (row stride free) . w [N, K]^T bf16
+void linear_f32(torch::Tensor out, torch::Tensor x, torch::Tensor w) {
+  check_small_linear(x, w);
+  CHECK_F32C(out);
+  const int T = x.size(0), N = w.size(0);
+  TORCH_CHECK(out.dim() == 2 && out.size(0) == T && out.size(1) == N);
+  launch_small_linear(out.data_ptr<float>(), x.data_ptr(), x.stride(0),
+                      w.data_ptr(), T, N, (int)x.size(1), nullptr, nullptr,
+                      nullptr, 0, 0, cur_stream());
+}
+
+// ids [T, top] int64, wts [T, top] fp32, rest [T, N - E] fp32
+void route_softmax(torch::Tensor ids, torch::Tensor wts, torch::Tensor rest,
+                   torch::Tensor x, torch::Tensor w, torch::Tensor bias,
+                   int64_t E, int64_t top) {
+  check_small_linear(x, w);
+  const int T = x.size(0), N = w.size(0);
+  TORCH_CHECK(E >= 1 && E <= N && N <= 240, "router rows");
+  TORCH_CHECK(top >= 1 && top <= E && top <= 64, "experts per token");
+  CHECK_I64(ids);
+  CHECK_F32C(wts);
+  CHECK_F32C(rest);
+  TORCH_CHECK(ids.numel() == T * top && wts.numel() == T * top &&
+              rest.numel() == (int64_t)T * (N - E));
+  const bool has_b = bias.numel() > 0;
+  if (has_b) {
+    CHECK_F32C(bias);
+    TORCH_CHECK(bias.numel() == E);
+  }
+  launch_small_linear(rest.data_ptr<float>(), x.data_ptr(), x.stride(0),
+                      w.data_ptr(), T, N, (int)x.size(1),
+                      ids.data_ptr<int64_t>(), wts.data_ptr<float>(),
+                      has_b ? bias.data_ptr<float>() : nullptr, (int)E,
+                      (int)top, cur_stream());
+}
+
+// q, k [T, H * d], v, g [T, H * dv] (row strides free), gates [T, 2 H] fp32,
+// gate_bias [2 H] fp32, norm_w [H * dv], state [slots, H, sw] fp32, slots [B]
+// int64, cu [B+1] int32 or empty (one token per sequence), out [T, H * dv]
+void mlstm(torch::Tensor out, torch::Tensor q, torch::Tensor k, torch::Tensor v,
+           torch::Tensor g, torch::Tensor gates, torch::Tensor gate_bias,
+           torch::Tensor norm_w, double cap, double eps, torch::Tensor state,
+           torch::Tensor slots, torch::Tensor cu, torch::Tensor positions) {
+  const int kind = kind_of(q, "q");
+  CHECK_F32C(state);
+  TORCH_CHECK(state.dim() == 3 && q.dim() == 2 && v.dim() == 2);
+  const int H = state.size(1), T = q.size(0);
+  TORCH_CHECK(q.size(1) % H == 0 && v.size(1) % H == 0, "head widths");
+  const int d = q.size(1) / H, dv = v.size(1) / H;
+  const int64_t sw = state.size(2);
+  TORCH_CHECK(sw >= (int64_t)d * dv + d + 1 && sw % 4 == 0, "state row width");
+  TORCH_CHECK(d <= 1024, "mlstm key width above 1024 is not supported");
+  TORCH_CHECK(dv <= 4096, "mlstm value width above 4096 is not supported");
+  for (const torch::Tensor* t : {&q, &k})
+    TORCH_CHECK(t->is_cuda() && t->scalar_type() == q.scalar_type() &&
+                t->dim() == 2 && t->size(0) == T && t->size(1) == H * d &&
+                t->stride(1) == 1);
+  for (const torch::Tensor* t : {&v, &g})
+    TORCH_CHECK(t->is_cuda() && t->scalar_type() == q.scalar_type() &&
+                t->dim() == 2 && t->size(0) == T && t->size(1) == H * dv &&
+                t->stride(1) == 1);
+  CHECK_F32C(gates);
+  CHECK_F32C(gate_bias);
+  TORCH_CHECK(gates.dim() == 2 && gates.size(0) == T && gates.size(1) == 2 * H &&
+              gate_bias.numel() == 2 * H && cap > 0);
+  TORCH_CHECK(norm_w.is_cuda() && norm_w.scalar_type() == q.scalar_type() &&
+              norm_w.is_contiguous() && norm_w.numel() == H * dv);
+  TORCH_CHECK(out.is_cuda() && out.scalar_type() == q.scalar_type() &&
+              out.is_contiguous() && out.dim() == 2 && out.size(0) == T &&
+              out.size(1) == H * dv);
+  CHECK_I64(slots);
+  CHECK_I32(positions);
+  TORCH_CHECK(positions.numel() == T);
+  const int B = slots.numel();
+  const bool has_cu = cu.numel() > 0;
+  if (has_cu) {
+    CHECK_I32(cu);
+    TORCH_CHECK(cu.numel() == B + 1);
+  } else {
+    TORCH_CHECK(B == T, "without cu every sequence brings one token");
+  }
+  int path = 0;
+  torch::Tensor o, nq, mm;
+  if (has_cu) {
+    const bool aligned =
+        d % 8 == 0 && dv % 8 == 0 && q.stride(0) % 8 == 0 &&
+        k.stride(0) % 8 == 0 && v.stride(0) % 8 == 0 &&
+        ((uintptr_t)q.data_ptr() % 16) == 0 &&
+        ((uintptr_t)k.data_ptr() % 16) == 0 && ((uintptr_t)v.data_ptr() % 16) == 0;
+    path = (kind == 0 && d <= 128 && aligned) ? 2 : 1;
+    o = torch::empty({(int64_t)T, H, dv}, state.options());
+    nq = torch::empty({(int64_t)T, H}, state.options());
+    mm = torch::empty({(int64_t)T, H}, state.options());
+  }
+  launch_mlstm(out.data_ptr(), path ? o.data_ptr<float>() : nullptr,
+               path ? nq.data_ptr<float>() : nullptr,
+               path ? mm.data_ptr<float>() : nullptr, q.data_ptr(), q.stride(0),
+               k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0),
+               g.data_ptr(), g.stride(0), gates.data_ptr<float>(),
+               gate_bias.data_ptr<float>(), norm_w.data_ptr(), (float)cap,
+               (float)eps, state.data_ptr<float>(), sw, slots.data_ptr<int64_t>(),
+               has_cu ? cu.data_ptr<int>() : nullptr, positions.data_ptr<int>(),
+               T, B, H, d, dv, 1.0f / std::sqrt((float)d), path, kind,
+               cur_stream());
+}
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("add_layernorm", &add_layernorm);
   m.def("latent_kv_store", &latent_kv_store);
@@ -858,4 +1111,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("pair_hash_embedding", &pair_hash_embedding);
   m.def("relu_squared", &relu_squared);
   m.def("rotate_heads", &rotate_heads);
+  m.def("hyper_rmsnorm", &hyper_rmsnorm);
+  m.def("embed_streams", &embed_streams);
+  m.def("biased_glu", &biased_glu);
+  m.def("softcap_logits", &softcap_logits);
+  m.def("linear_f32", &linear_f32);
+  m.def("route_softmax", &route_softmax);
+  m.def("mlstm", &mlstm);
 }

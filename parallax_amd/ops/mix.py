@@ -4,7 +4,8 @@ RMS norm with depth-weighted averaging, row-cache attention (differential /
 pooled sliding window / sigmoid-weighted with an output gate) and xIELU;
 post-norm residual step, minGRU scan and the clamped gated linear unit;
 grouped RMS norm over a parallel residual, hashed pair embedding, squared relu
-and the rotation of head rows by position.
+and the rotation of head rows by position; hyper-connected residual streams,
+matrix LSTM, softmax router, biased gated linear unit.
 
 GPU tensors go to the hand-written gfx950 kernels of the in-tree extension
 ``parallax_amd.ops._mix`` (bf16 or float32 activations; scores, norms, decays
@@ -73,46 +74,61 @@ def add_layernorm(resid, y, scale, mult, weight, bias, eps, out_dtype):
 
 
 def latent_kv_store(dkv, norm_w, eps, freq, mult, rot_dims, positions,
-                    slot_mapping, cache, rank):
-    """RMS-norm the first `rank` columns of dkv, rotate the rest by position,
-    scatter both as one cache row per token (slot -1 = skip)."""
+                    slot_mapping, cache, rank, interleaved=False, q_down=None,
+                    q_norm_w=None):
+    """RMS-norm the first `rank` columns of dkv, rotate the rest by position
+    (pairs i, i + rot_dims/2, or 2i, 2i + 1 when interleaved), scatter both as
+    one cache row per token (slot -1 = skip). q_down [T, q_rank] given: the
+    same launch RMS-norms it with weight q_norm_w and returns the result."""
     if not dkv.is_cuda:
         return ref.latent_kv_store(dkv, norm_w, eps, freq, mult, rot_dims,
-                                   positions, slot_mapping, cache, rank)
+                                   positions, slot_mapping, cache, rank,
+                                   interleaved, q_down, q_norm_w)
+    e = _empty(dkv)
+    q_out = torch.empty(q_down.shape, dtype=q_down.dtype, device=dkv.device) \
+        if q_down is not None else None
     _mix_ext().latent_kv_store(dkv, norm_w, float(eps), freq, float(mult),
                                int(rot_dims), positions, slot_mapping, cache,
-                               int(rank))
+                               int(rank), bool(interleaved),
+                               q_down if q_down is not None else e,
+                               q_norm_w if q_down is not None else e,
+                               q_out if q_down is not None else e)
+    return q_out
 
 
-def rope_rows(q, col0, rot_w, freq, mult, rot_dims, positions):
+def rope_rows(q, col0, rot_w, freq, mult, rot_dims, positions, interleaved=False):
     """q [T, H, D]: columns [col0, col0+rot_w) of every head, rotated on their
-    first rot_dims dimensions, as a new fp32 [T, H, rot_w]."""
+    first rot_dims dimensions (either pairing), as a new fp32 [T, H, rot_w]."""
     if not q.is_cuda:
-        return ref.rope_rows(q, col0, rot_w, freq, mult, rot_dims, positions)
+        return ref.rope_rows(q, col0, rot_w, freq, mult, rot_dims, positions,
+                             interleaved)
     out = torch.empty(q.shape[0], q.shape[1], rot_w, dtype=torch.float32,
                       device=q.device)
     _mix_ext().rope_rows(out, q, int(col0), freq, float(mult), int(rot_dims),
-                         positions)
+                         positions, bool(interleaved))
     return out
 
 
 def latent_window_attention(q_lat, q_rot, cache, block_tables, token_seq,
-                            positions, window, scale, max_seq_len=0):
+                            positions, window, scale, max_seq_len=0, sink=None):
     """Softmax attention of absorbed queries over the paged latent cache with
     a sliding window: token at position p sees keys p-window+1 .. p of its
     sequence. q_lat [T, H, rank] fp32, q_rot [T, H, rot_w] fp32, token_seq [T]
     int32 (None: token i is sequence i). max_seq_len: the longest context in
     the batch as the host knows it (0 = the block tables' capacity); it only
-    sizes the split of long windows over workgroups. Returns fp32 [T, H, rank]."""
+    sizes the split of long windows over workgroups. sink [H] fp32: the
+    softmax's denominator also holds exp(sink[h]). Returns fp32 [T, H, rank]."""
     if not q_lat.is_cuda:
         return ref.latent_window_attention(q_lat, q_rot, cache, block_tables,
-                                           token_seq, positions, window, scale)
+                                           token_seq, positions, window, scale,
+                                           sink)
     out = torch.empty_like(q_lat)
     _mix_ext().latent_window_attention(
         out, q_lat, q_rot, cache, block_tables,
         token_seq if token_seq is not None
         else _empty(positions), positions, int(window), float(scale),
         int(max_seq_len) or block_tables.shape[1] * cache.shape[1],
+        sink if sink is not None else _empty(q_lat),
     )
     return out
 
@@ -411,4 +427,133 @@ def rotate_heads(x, positions, freq, interleaved, sign, out_dtype):
     out = torch.empty(T, H * D, dtype=out_dtype, device=x.device)
     _mix_ext().rotate_heads(out, x.contiguous(), freq, positions,
                             bool(interleaved), float(sign))
+    return out
+
+
+# -- hyper-connections, matrix LSTM, routed experts' front end ---------------------
+
+
+def embed_streams(ids, table, streams):
+    """fp32 [T, streams * W]: table[id], once per residual stream."""
+    if not table.is_cuda:
+        return ref.embed_streams(ids, table, streams)
+    out = torch.empty(ids.shape[0], streams * table.shape[1],
+                      dtype=torch.float32, device=table.device)
+    _mix_ext().embed_streams(out, ids, table, int(streams))
+    return out
+
+
+def hyper_rmsnorm(x, y, y_bias, y2, gate2, mix, out_w, in_w, weight, eps,
+                  out_dtype):
+    """One residual step over S hyper-connected streams, one kernel; x [T, S *
+    W] fp32 (in place):
+      z = y + y_bias + sigmoid(gate2) * y2   (y_bias, y2 + gate2 [T] optional)
+      x_t <- sum_s mix[s, t] x_s + out_w[t] z,  all streams from the old ones
+             (y None: no update)
+      u = sum_s in_w[s] x_s;  returns u / sqrt(mean(u^2) + eps) * weight in
+      out_dtype (in_w None: no read, returns None)
+    mix [S, S], out_w [S], in_w [S] fp32; y, y2 in the activation dtype or
+    fp32 each."""
+    if not x.is_cuda:
+        return ref.hyper_rmsnorm(x, y, y_bias, y2, gate2, mix, out_w, in_w,
+                                 weight, eps, out_dtype)
+    S = (in_w if in_w is not None else out_w).shape[0]
+    T, W = x.shape[0], x.shape[1] // S
+    ef, e = _empty(x), _empty(x, out_dtype)
+    out = torch.empty(T, W, dtype=out_dtype, device=x.device) \
+        if in_w is not None else e
+    has = y is not None
+    _mix_ext().hyper_rmsnorm(
+        x, y if has else e, y_bias if has and y_bias is not None else e,
+        y2 if has and y2 is not None else e,
+        gate2 if has and y2 is not None else ef,
+        mix if has else ef, out_w if has else ef,
+        in_w if in_w is not None else ef,
+        weight if in_w is not None else e, float(eps), out, int(S),
+    )
+    return out if in_w is not None else None
+
+
+def mlstm(q, k, v, g, gates, gate_bias, norm_w, cap, eps, state, slots, cu,
+          positions, out_dtype):
+    """Matrix LSTM over packed sequences with per-head RMS norm and sigmoid
+    output gate (see reference.mlstm for the equations). q, k [T, H * d] and
+    v, g [T, H * dv] (row strides free); gates [T, 2 H] fp32 pre-activations
+    [input | forget], gate_bias [2 H] fp32; norm_w [H * dv]; the fp32 state
+    [slots, H, >= d dv + d + 1] is read (or started from zero at position 0)
+    and written back. cu [B+1] int32 token bounds (None: one token each).
+    Returns [T, H * dv] of out_dtype."""
+    if not q.is_cuda:
+        return ref.mlstm(q, k, v, g, gates, gate_bias, norm_w, cap, eps, state,
+                         slots, cu, positions, out_dtype)
+    out = torch.empty(q.shape[0], v.shape[1], dtype=out_dtype, device=q.device)
+    _mix_ext().mlstm(
+        out, q, k, v, g, gates, gate_bias, norm_w, float(cap), float(eps),
+        state, slots, cu if cu is not None else _empty(positions), positions,
+    )
+    return out
+
+
+def linear_f32(x, weight):
+    """x [T, W] @ weight [N, W]^T with an fp32 result, for the few columns
+    (gates, router logits) whose consumers want more than bf16."""
+    if not x.is_cuda:
+        return ref.linear_f32(x, weight)
+    if x.dtype == torch.float32:
+        return torch.nn.functional.linear(x, weight)
+    out = torch.empty(x.shape[0], weight.shape[0], dtype=torch.float32,
+                      device=x.device)
+    _mix_ext().linear_f32(out, x, weight)
+    return out
+
+
+ROUTE_MAX_ROWS = 240   # rows of the routing kernel's weight
+ROUTE_MAX_TOP = 64     # experts it chooses per token
+
+
+def route_softmax(x, weight, bias, experts, top):
+    """Router: z = x W[:experts]^T + bias in fp32, the `top` largest, weights =
+    softmax over those; rows of weight after the experts come back as plain
+    fp32 outputs. One kernel for bf16 activations and up to ROUTE_MAX_ROWS
+    rows. Returns (ids [T, top] int64, weights [T, top] fp32, rest [T, N -
+    experts] fp32). bias [experts] fp32 or None."""
+    if not x.is_cuda:
+        return ref.route_softmax(x, weight, bias, experts, top)
+    T, N = x.shape[0], weight.shape[0]
+    if x.dtype == torch.float32 or N > ROUTE_MAX_ROWS or top > ROUTE_MAX_TOP:
+        z = linear_f32(x, weight)
+        zr = z[:, :experts] if bias is None else z[:, :experts] + bias
+        val, ids = zr.topk(top, dim=-1)
+        return ids, torch.softmax(val, dim=-1), z[:, experts:].contiguous()
+    ids = torch.empty(T, top, dtype=torch.int64, device=x.device)
+    wts = torch.empty(T, top, dtype=torch.float32, device=x.device)
+    rest = torch.empty(T, N - experts, dtype=torch.float32, device=x.device)
+    _mix_ext().route_softmax(ids, wts, rest, x, weight,
+                             bias if bias is not None else _empty(wts),
+                             int(experts), int(top))
+    return ids, wts, rest
+
+
+def biased_glu(gate_up, bias, act):
+    """[gate | up] (+ bias [2 I]) -> act(gate) * up, fp32 inside, result in the
+    input dtype. act: 'silu' or 'gelu_tanh'. gate_up may be a column range of
+    a wider matrix."""
+    if act not in ("silu", "gelu_tanh"):
+        raise ValueError(f"unknown activation {act!r}")
+    if not gate_up.is_cuda:
+        return ref.biased_glu(gate_up, bias, act)
+    out = torch.empty(gate_up.shape[0], gate_up.shape[1] // 2,
+                      dtype=gate_up.dtype, device=gate_up.device)
+    _mix_ext().biased_glu(out, gate_up,
+                          bias if bias is not None else _empty(gate_up),
+                          act == "gelu_tanh")
+    return out
+
+
+def softcap_logits(x, scale, cap):
+    """fp32 logits: z = x * scale; cap > 0: cap * tanh(z / cap)."""
+    if not x.is_cuda:
+        return ref.softcap_logits(x, scale, cap)
+    out = torch.empty(x.shape, dtype=torch.float32, device=x.device)
+    _mix_ext().softcap_logits(out, x.contiguous(), float(scale), float(cap))
     return out

@@ -599,26 +599,33 @@ def _rotate_rows(x, positions, freq, mult, rot_dims, interleaved=False,
 
 
 def latent_kv_store(dkv, norm_w, eps, freq, mult, rot_dims, positions,
-                    slot_mapping, cache, rank):
+                    slot_mapping, cache, rank, interleaved=False, q_down=None,
+                    q_norm_w=None):
+    """q_down [T, q_rank] given: also returns its RMS norm times q_norm_w."""
     x = dkv.float()
     lat = x[:, :rank]
     lat = lat / torch.sqrt((lat * lat).mean(-1, keepdim=True) + eps) * norm_w.float()
     kr = x[:, rank:]
     if rot_dims > 0:
-        kr = _rotate_rows(kr, positions, freq, mult, rot_dims)
+        kr = _rotate_rows(kr, positions, freq, mult, rot_dims, interleaved)
     entry = torch.cat([lat, kr], dim=-1).to(cache.dtype)
     keep = slot_mapping >= 0
     flat = cache.view(-1, cache.shape[-1])
     flat[slot_mapping[keep]] = entry[keep]
+    if q_down is None:
+        return None
+    q = q_down.float()
+    q = q / torch.sqrt((q * q).mean(-1, keepdim=True) + eps) * q_norm_w.float()
+    return q.to(q_down.dtype)
 
 
-def rope_rows(q, col0, rot_w, freq, mult, rot_dims, positions):
+def rope_rows(q, col0, rot_w, freq, mult, rot_dims, positions, interleaved=False):
     return _rotate_rows(q[..., col0 : col0 + rot_w].float(), positions, freq,
-                        mult, rot_dims).contiguous()
+                        mult, rot_dims, interleaved).contiguous()
 
 
 def latent_window_attention(q_lat, q_rot, cache, block_tables, token_seq,
-                            positions, window, scale):
+                            positions, window, scale, sink=None):
     T, H, rank = q_lat.shape
     bs = cache.shape[1]
     out = torch.empty_like(q_lat)
@@ -631,7 +638,9 @@ def latent_window_attention(q_lat, q_rot, cache, block_tables, token_seq,
         bt = block_tables[seq[t]].long()
         rows = cache[bt[j // bs], j % bs].float()                  # [n, E]
         s = (q_lat[t] @ rows[:, :rank].T + q_rot[t] @ rows[:, rank:].T) * scale
-        out[t] = torch.softmax(s, dim=-1) @ rows[:, :rank]
+        if sink is not None:   # a key-less term of the denominator
+            s = torch.cat([s, sink.float().view(H, 1)], dim=-1)
+        out[t] = torch.softmax(s, dim=-1)[:, : p - lo + 1] @ rows[:, :rank]
     return out
 
 
@@ -994,3 +1003,126 @@ def relu_squared(x):
     """max(x, 0)^2 (fp32 inside, result in the input dtype)."""
     z = x.float().clamp(min=0.0)
     return (z * z).to(x.dtype)
+
+
+# -- hyper-connections, matrix LSTM, routed experts' front end ---------------------
+
+
+def embed_streams(ids, table, streams):
+    """fp32 [T, streams * W]: the token's row, once per stream."""
+    return table[ids.long()].float().repeat(1, streams)
+
+
+def hyper_rmsnorm(x, y, y_bias, y2, gate2, mix, out_w, in_w, weight, eps,
+                  out_dtype):
+    """One residual step over S streams, x [T, S * W] fp32 in place:
+      z = y + y_bias + sigmoid(gate2) * y2          (what is given of it)
+      x_t <- sum_s mix[s, t] x_s + out_w[t] * z     (all streams from the old
+                                                     ones; y None: no update)
+      u = sum_s in_w[s] x_s,   h = u / sqrt(mean(u^2) + eps) * weight
+    Returns h in out_dtype (None when in_w is None)."""
+    T = x.shape[0]
+    S = (in_w if in_w is not None else out_w).shape[0]
+    X = x.view(T, S, -1)
+    if y is not None:
+        z = y.float()
+        if y_bias is not None:
+            z = z + y_bias.float()
+        if y2 is not None:
+            z = z + torch.sigmoid(gate2.float()).view(T, 1) * y2.float()
+        new = torch.einsum("st,nsw->ntw", mix.float(), X) \
+            + out_w.float().view(1, S, 1) * z.unsqueeze(1)
+        X.copy_(new)
+    if in_w is None:
+        return None
+    u = torch.einsum("s,nsw->nw", in_w.float(), X)
+    h = u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * weight.float()
+    return h.to(out_dtype)
+
+
+def mlstm(q, k, v, g, gates, gate_bias, norm_w, cap, eps, state, slots, cu,
+          positions, out_dtype):
+    """Matrix LSTM over packed sequences. q, k [T, H * d], v, g [T, H * dv],
+    gates [T, 2 H] = [input | forget] pre-activations, gate_bias [2 H],
+    state [slots, H, >= d * dv + d + 1] fp32 holding per head the matrix
+    [d, dv], the normaliser [d] and the running maximum. Per head and token
+      i = cap tanh(i_pre / cap),  f = logsigmoid(cap tanh(f_pre / cap)),
+      m' = max(f + m, i),  a = exp(f + m - m'),  b = exp(i - m'),
+      S <- a S + b k v^T,  n <- a n + b k,
+      o = S^T q / (max(|n . q|, exp(-m')) + 1e-6)   with q scaled by d^-1/2;
+    then o / rms(o) * norm_w * sigmoid(g), all of it fp32. A portion that
+    starts at position 0 starts from zeros. Returns [T, H * dv]."""
+    T = q.shape[0]
+    H = state.shape[1]
+    d, dv = q.shape[1] // H, v.shape[1] // H
+    qf = q.float().view(T, H, d) * d ** -0.5
+    kf = k.float().view(T, H, d)
+    vf = v.float().view(T, H, dv)
+    z = cap * torch.tanh((gates.float() + gate_bias.float()) / cap)
+    gi, gf = z[:, :H], torch.nn.functional.logsigmoid(z[:, H:])
+    o = torch.empty(T, H, dv, dtype=torch.float32)
+    bounds = cu.tolist() if cu is not None else list(range(T + 1))
+    pos = positions.tolist()
+    for b, slot in enumerate(slots.tolist()):
+        t0, t1 = bounds[b], bounds[b + 1]
+        if t0 >= t1:
+            continue
+        row = state[slot]
+        if pos[t0] == 0:
+            row.zero_()
+        S = row[:, : d * dv].reshape(H, d, dv).clone()
+        n = row[:, d * dv : d * dv + d].clone()
+        m = row[:, d * dv + d].clone()
+        for t in range(t0, t1):
+            m_new = torch.maximum(gf[t] + m, gi[t])
+            a = torch.exp(gf[t] + m - m_new)
+            bb = torch.exp(gi[t] - m_new)
+            m = m_new
+            kb = bb.view(H, 1) * kf[t]
+            S = a.view(H, 1, 1) * S + kb.unsqueeze(-1) * vf[t].unsqueeze(-2)
+            n = a.view(H, 1) * n + kb
+            den = torch.maximum((n * qf[t]).sum(-1).abs(), torch.exp(-m)) + 1e-6
+            o[t] = torch.einsum("hkv,hk->hv", S, qf[t]) / den.view(H, 1)
+        row[:, : d * dv] = S.reshape(H, d * dv)
+        row[:, d * dv : d * dv + d] = n
+        row[:, d * dv + d] = m
+    o = o / torch.sqrt((o * o).mean(-1, keepdim=True) + eps)
+    o = o.view(T, H * dv) * norm_w.float() * torch.sigmoid(g.float())
+    return o.to(out_dtype)
+
+
+def linear_f32(x, weight):
+    """x [T, W] @ weight [N, W]^T with an fp32 result."""
+    return x.float() @ weight.float().t()
+
+
+def route_softmax(x, weight, bias, experts, top):
+    """Router over the first `experts` rows of weight [N, W], N >= experts:
+    the `top` largest of z = x W^T + bias, weights = softmax over those; the
+    rows after the experts are plain fp32 outputs. Returns (ids [T, top]
+    int64, weights [T, top] fp32, rest [T, N - experts] fp32)."""
+    z = linear_f32(x, weight)
+    zr = z[:, :experts]
+    if bias is not None:
+        zr = zr + bias.float()
+    val, ids = zr.topk(top, dim=-1)
+    return ids, torch.softmax(val, dim=-1), z[:, experts:].contiguous()
+
+
+def biased_glu(gate_up, bias, act):
+    """[gate | up] (+ bias) -> act(gate) * up, fp32 inside, result in the
+    input dtype. act: 'silu' or 'gelu_tanh'."""
+    z = gate_up.float()
+    if bias is not None:
+        z = z + bias.float()
+    I = z.shape[-1] // 2
+    a = z[..., :I]
+    a = torch.nn.functional.silu(a) if act == "silu" \
+        else torch.nn.functional.gelu(a, approximate="tanh")
+    return (a * z[..., I:]).to(gate_up.dtype)
+
+
+def softcap_logits(x, scale, cap):
+    """fp32: z = x * scale; cap > 0: cap * tanh(z / cap)."""
+    z = x.float() * scale
+    return cap * torch.tanh(z / cap) if cap > 0 else z

@@ -133,6 +133,9 @@ class Engine:
         # dtype of the hidden states that enter and leave a shard (designs
         # that keep their residual stream in fp32 say so on the model class)
         self.hidden_dtype = getattr(self.model, "hidden_dtype", None) or args.dtype
+        # and their width per token (stacks with several residual streams
+        # hand all of them on)
+        self.hidden_width = int(getattr(self.model, "hidden_width", cfg.hidden_size))
         # models whose embedding reads the (previous token, token) pair get
         # every token's predecessor in ForwardMeta.prev_ids
         self.uses_prev_tokens = bool(getattr(self.model, "uses_prev_tokens", False))
@@ -274,7 +277,7 @@ class Engine:
             self.graph_runner = DecodeGraphRunner(
                 self.model, self.kv_cache, self.device, self.hidden_dtype,
                 max_batch=args.max_batch_size, max_model_len=args.max_model_len,
-                block_size=args.block_size, hidden_size=cfg.hidden_size,
+                block_size=args.block_size, hidden_size=self.hidden_width,
                 is_first_stage=self.comm.is_first_stage,
                 is_last_stage=self.comm.is_last_stage,
                 is_mla=self.is_mla,
@@ -868,7 +871,7 @@ class Engine:
         on the last stage, None elsewhere."""
         comm = self.comm
         T = meta.num_tokens
-        h = self.cfg.hidden_size
+        h = self.hidden_width
         if comm.is_first_stage:
             hidden = self._embed(input_ids, meta)
         else:
@@ -897,7 +900,7 @@ class Engine:
             # hidden states for group g-1 are in flight to stage i+1 (same
             # pre-posted-irecv + staged-isend pattern as _run_decode)
             comm = self.comm
-            h = self.cfg.hidden_size
+            h = self.hidden_width
             recvs: List[tuple] = []
             if not comm.is_first_stage:
                 for g in groups:
@@ -999,7 +1002,7 @@ class Engine:
         hidden_in = None
         if not comm.is_first_stage:
             hidden_in = comm.pp_recv(
-                (len(reqs), self.cfg.hidden_size), self.hidden_dtype, comm.pp_rank - 1
+                (len(reqs), self.hidden_width), self.hidden_dtype, comm.pp_rank - 1
             )
         out = self._decode_fwd(reqs, hidden_in)
         if not comm.is_last_stage:
@@ -1019,7 +1022,7 @@ class Engine:
             # states are still in flight over xGMI.
             groups: List[List[InitialRequest]] = [list(x) for x in _split(reqs, mb)]
             comm = self.comm
-            h = self.cfg.hidden_size
+            h = self.hidden_width
             recvs: List[tuple] = []
             if not comm.is_first_stage:
                 for g in groups:

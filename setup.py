@@ -5,7 +5,8 @@
 The built .so files land at parallax_amd/ops/_C.*.so (attention, GEMM, MoE,
 sampler kernels) and parallax_amd/ops/_mix.*.so (sequence mixers: fp32-residual
 layer norm, sliding-window latent attention, gated linear attention, sandwich
-RMS norm, row-cache attention, post-norm residual step, minGRU). Both are
+RMS norm, row-cache attention, post-norm residual step, minGRU, hyper-connected
+streams, matrix LSTM, softmax router). Both are
 git-ignored; they travel to the GPU box with the gpurun snapshot.
 PARALLAX_EXT=_mix (or _C) builds one of them only.
 """
@@ -55,6 +56,9 @@ mix_sources = [
     os.path.join(CSRC, "row_attention_mfma.hip"),
     os.path.join(CSRC, "post_norm.hip"),
     os.path.join(CSRC, "group_norm.hip"),
+    os.path.join(CSRC, "hyper.hip"),
+    os.path.join(CSRC, "small_linear.hip"),
+    os.path.join(CSRC, "mlstm.hip"),
 ]
 
 wanted = [x for x in os.environ.get("PARALLAX_EXT", "_C,_mix").split(",") if x]
