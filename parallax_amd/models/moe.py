@@ -299,7 +299,10 @@ class FusedMoE(nn.Module):
                 gate = h[:, :I].clamp(max=self.act_limit)
                 up = h[:, I:].clamp(min=-self.act_limit, max=self.act_limit)
                 h = ((up + 1.0) * (gate * torch.sigmoid(gate * 1.702))).to(xe.dtype)
-            elif (h.is_cuda and h.dtype != torch.bfloat16) or self.weight_on_input:
+            elif h.is_cuda and not self.weight_on_input and (
+                    h.dtype != torch.bfloat16 or self.intermediate_size % 8):
+                h = ops.biased_glu(h, None, "silu")
+            elif self.weight_on_input:
                 I = self.intermediate_size
                 h = (F.silu(h[:, :I]) * h[:, I:]).to(xe.dtype)
             else:

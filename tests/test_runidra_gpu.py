@@ -1,0 +1,179 @@
+"""Runidra on the GPU engine (HIP kernels, bf16 and float32) against the plain
+reference in runidra_oracle.py: mixed batches, portions, decoding through
+hipGraphs, pages and state slots used again, irregular sizes, greedy
+generation."""
+
+import pytest
+import torch
+
+import runidra_oracle as oracle
+import runidra_util as U
+from parallax_amd import ops
+from parallax_amd.server.sampling_params import SamplingParams
+
+pytestmark = pytest.mark.gpu
+
+TOL = {torch.float32: 3e-4, torch.bfloat16: 0.08}
+
+
+def close(got, want, dtype) -> bool:
+    """float32: every row within rounding of the float64 reference. bfloat16:
+    router near-ties and head norms over cancelling sums make single rows far
+    more sensitive to rounding than the rest, and a flipped choice stays in
+    the recurrent state: 85 rows in 100 within 0.08 and the median under 0.04;
+    same_as_whole() is the sharp bf16 check."""
+    if dtype == torch.bfloat16:
+        e = U.row_errs(got, want)
+        few = e.numel() < 8          # a median of a handful of rows says little
+        return bool((e < TOL[dtype]).double().mean() >= 0.85
+                    and (few or e.median() < 0.04))
+    return U.rel_err(got, want) < TOL[dtype]
+
+
+@pytest.fixture(scope="module")
+def ckpt(tmp_path_factory):
+    # widths on the vector and matrix-core paths (multiples of 8) and off them
+    # (12 / 20), expert widths the grouped-GEMM kernels tile (32, 96)
+    layers = [
+        U.mlstm_layer(),
+        U.latent_layer(mlp=U.experts(5, 2, 32, 40)),
+        U.mlstm_layer(2, 40, 72, 15.0, None),
+        U.latent_layer(4, 8, 8, 16, 40, 24, 33, 0.4, 10000.0, U.dense(64)),
+        U.mlstm_layer(1, 16, 16, 4.0, U.experts(3, 1, 96, 0)),
+    ]
+    cfg = U.small_config(layers, width=64, vocab=136)
+    w = oracle.random_weights(cfg, seed=3)
+    path = U.write_checkpoint(str(tmp_path_factory.mktemp("rng")), cfg, w)
+    return cfg, w, path
+
+
+SEQS = {"a": (90, 4), "b": (7, 5), "c": (41, 6), "d": (1, 7), "e": (30, 8)}
+SCHEDULE = [
+    [("a", 16), ("b", 1)],
+    [("b", 1), ("a", 31), ("c", 2)],
+    [("c", 1), ("b", 1), ("a", 1), ("d", 1)],
+    [("e", 9), ("a", 1), ("b", 4), ("c", 30)],
+    [("a", 40), ("c", 1), ("e", 1)],
+    [("e", 20), ("a", 1), ("c", 7)],
+]
+
+
+@pytest.mark.parametrize("dtype,graphs", [(torch.float32, False), (torch.bfloat16, False),
+                                          (torch.bfloat16, True)])
+def test_mixed_batches(ckpt, dtype, graphs):
+    cfg, w, path = ckpt
+    assert ops.has_mix_extension()
+    seqs = {k: U.tokens(n, cfg["vocab"], s) for k, (n, s) in SEQS.items()}
+    eng = U.make_engine(path, device="cuda", dtype=dtype, pages=24, graphs=graphs)
+    assert (eng.graph_runner is not None) == graphs
+    got = U.run_schedule(eng, seqs, SCHEDULE)
+    alone = U.make_engine(path, device="cuda", dtype=dtype, pages=24)
+    for name, toks in seqs.items():
+        want = oracle.forward(cfg, w, toks)
+        assert close(got[name], want, dtype), (name, U.describe(got[name], want, TOL[dtype]))
+        whole = U.run_schedule(alone, {name: toks}, [[(name, len(toks))]])[name]
+        assert U.same_as_whole(got[name], whole, 0.05), (name, U.describe(got[name], whole, 0.05))
+    assert eng.cache_manager.num_free_blocks == 24
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_portions_decoding_and_reuse(ckpt, dtype):
+    cfg, w, path = ckpt
+    eng = U.make_engine(path, device="cuda", dtype=dtype, pages=20, max_requests=2,
+                        graphs=dtype == torch.bfloat16)
+    alone = U.make_engine(path, device="cuda", dtype=dtype, pages=20)
+    for k, cuts in enumerate([[150], [2] * 20 + [1] * 60, [3, 2, 7, 1, 1, 1, 33, 2, 5, 45],
+                              [12] + [1] * 128]):
+        toks = U.tokens(sum(cuts), cfg["vocab"], 40 + k)
+        got = U.run_schedule(eng, {"r": toks}, [[("r", n)] for n in cuts])["r"]
+        want = oracle.forward(cfg, w, toks)
+        assert close(got, want, dtype), (cuts[:3], U.describe(got, want, TOL[dtype]))
+        whole = U.run_schedule(alone, {"w": toks}, [[("w", len(toks))]])["w"]
+        assert U.same_as_whole(got, whole, 0.05), (cuts[:3], U.describe(got, whole, 0.05))
+        assert eng.cache_manager.num_free_blocks == 20
+
+
+def test_cutting_changes_nothing_beyond_rounding(ckpt):
+    cfg, w, path = ckpt
+    toks = U.tokens(100, cfg["vocab"], 50)
+    eng = U.make_engine(path, device="cuda", dtype=torch.float32)
+    whole = U.run_schedule(eng, {"a": toks}, [[("a", 100)]])["a"]
+    cut = U.run_schedule(eng, {"b": toks}, [[("b", n)] for n in [37, 1, 1, 2, 59]])["b"]
+    assert U.rel_err(cut, whole.double()) < 1e-4
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_sizes_outside_the_tuned_paths(tmp_path, dtype):
+    """A width, vocabulary, head and expert sizes that are no multiples of 8:
+    vendor's plain GEMM, scalar paths of the kernels, token-serial matrix
+    LSTM, per-expert loop (decode then runs eagerly)."""
+    layers = [U.mlstm_layer(3, 10, 6, 5.0, U.dense(20)),
+              U.latent_layer(5, 12, 6, 10, 13, 7, 11, mlp=U.experts(3, 2, 20, 14)),
+              U.mlstm_layer(1, 21, 9, 9.0, None)]
+    cfg = U.small_config(layers, width=46, vocab=53, streams=5, loop=(1, 3, 2))
+    w = oracle.random_weights(cfg, seed=17)
+    path = U.write_checkpoint(str(tmp_path), cfg, w)
+    eng = U.make_engine(path, device="cuda", dtype=dtype, graphs=dtype == torch.bfloat16)
+    assert eng.graph_runner is None     # the per-expert loop reads the routing on the host
+    toks = U.tokens(75, 53, 10)
+    got = U.run_schedule(eng, {"a": toks},
+                         [[("a", n)] for n in [6, 1, 1, 30, 2, 5] + [1] * 30])["a"]
+    want = oracle.forward(cfg, w, toks)
+    assert close(got, want, dtype), U.describe(got, want, TOL[dtype])
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_long_contexts_and_wide_heads(tmp_path, dtype):
+    """Head widths, latents and windows of a real model's size beside small
+    ones, contexts of many pages and chunks: long portions take the tiled
+    kernels, single tokens the decode ones, and all agree with the
+    reference."""
+    layers = [U.latent_layer(8, 64, 32, 64, 256, 96, 200, 0.1, 40000.0, U.dense(128)),
+              U.mlstm_layer(2, 128, 128, 15.0, U.experts(6, 2, 96, 64)),
+              U.latent_layer(16, 128, 64, 128, 512, 192, 333, 0.07, 10000.0, None),
+              U.mlstm_layer(3, 64, 104, 8.0, None)]
+    cfg = U.small_config(layers, width=128, vocab=216, streams=2, loop=(1, 3, 2))
+    w = oracle.random_weights(cfg, seed=23)
+    path = U.write_checkpoint(str(tmp_path), cfg, w)
+    eng = U.make_engine(path, device="cuda", dtype=dtype, pages=40, block_size=32,
+                        graphs=dtype == torch.bfloat16)
+    seqs = {"a": U.tokens(700, 216, 31), "b": U.tokens(235, 216, 32)}
+    schedule = [[("a", 333)], [("a", 300), ("b", 200)], [("a", 1), ("b", 1)],
+                [("a", 36), ("b", 4)]] + [[("a", 1), ("b", 1)]] * 30
+    got = U.run_schedule(eng, seqs, schedule)
+    for name, toks in seqs.items():
+        want = oracle.forward(cfg, w, toks)
+        assert close(got[name], want, dtype), (name, U.describe(got[name], want, TOL[dtype]))
+
+
+def test_greedy_generation_fp32_matches_the_reference(ckpt):
+    cfg, w, path = ckpt
+    eng = U.make_engine(path, device="cuda", dtype=torch.float32, prefill_chunk_size=16)
+    prompts = [U.tokens(37, cfg["vocab"], 11), U.tokens(5, cfg["vocab"], 12)]
+    sp = [SamplingParams(temperature=0.0, max_new_tokens=n, ignore_eos=True) for n in (10, 16)]
+    out = list(eng.generate(prompts, sp).values())
+    for p, s, got in zip(prompts, sp, out):
+        seq = list(p)
+        for _ in range(s.max_new_tokens):
+            seq.append(int(oracle.forward(cfg, w, seq)[-1].argmax()))
+        assert got == seq[len(p):]
+
+
+def test_greedy_generation_bf16_through_graphs(ckpt):
+    """bf16 + captured decode graphs + async decode: every generated token is
+    the reference's best token or within rounding of it."""
+    cfg, w, path = ckpt
+    eng = U.make_engine(path, device="cuda", dtype=torch.bfloat16, graphs=True)
+    eng.warmup_serving()   # what `serve` does at start: GEMM picks, every decode graph
+    prompts = [U.tokens(29, cfg["vocab"], 21), U.tokens(3, cfg["vocab"], 22),
+               U.tokens(64, cfg["vocab"], 23)]
+    sp = [SamplingParams(temperature=0.0, max_new_tokens=24, ignore_eos=True)] * 3
+    out = list(eng.generate(prompts, sp).values())
+    for p, got in zip(prompts, out):
+        assert len(got) == 24
+        logits = oracle.forward(cfg, w, list(p) + got)
+        spread = float(logits.std())
+        for i, tok in enumerate(got):
+            row = logits[len(p) - 1 + i]
+            assert float(row.max() - row[tok]) < 0.25 * spread, (i, tok)
+    assert eng.cache_manager.num_free_blocks == 64
