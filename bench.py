@@ -364,6 +364,51 @@ def qwen3_like_pudizen_config(z: dict) -> dict:
     return cfg
 
 
+# `--design-compare --design-pair runidra`: a Runidra stack (matrix LSTM and
+# windowed latent attention with a query latent and sinks, two hyper-connected
+# streams, routed experts) beside a Vurizen stack (gated linear attention and
+# windowed latent attention, routed experts) of EQUAL sizes: the same head,
+# latent and window sizes, the same experts, recurrent and attention layers in
+# turn. No loop and no shared expert here, so that both do the same work a layer.
+
+RUNIDRA_SIZES = {
+    "s": dict(width=1024, layers=8, heads=8, nope=64, rot=64, vdim=64, rank=512,
+              q_rank=512, window=1024, experts=16, top=2, ff=512, streams=2,
+              groups=1, keep=1, vocab=32000),
+    "m": dict(width=2048, layers=8, heads=16, nope=128, rot=64, vdim=128, rank=512,
+              q_rank=1024, window=1024, experts=32, top=4, ff=1024, streams=2,
+              groups=1, keep=1, vocab=32000),
+    "l": dict(width=4096, layers=8, heads=32, nope=128, rot=64, vdim=128, rank=512,
+              q_rank=1536, window=1024, experts=32, top=4, ff=1024, streams=4,
+              groups=1, keep=1, vocab=32000),
+}
+
+
+def runidra_config(z: dict) -> dict:
+    mlp = {"kind": "moe", "expert": {"ff": z["ff"]},
+           "router": {"experts": z["experts"], "top": z["top"]}}
+    latent = {"type": "latent_attention", "mlp": mlp, "mixer": {
+        "heads": z["heads"], "dim": z["nope"], "rot_dim": z["rot"], "vdim": z["vdim"],
+        "kv_rank": z["rank"], "q_rank": z["q_rank"], "mask": {"size": z["window"]},
+        "scale": (z["nope"] + z["rot"]) ** -0.5,
+        "rot": {"dims": z["rot"], "base": 10000.0}}}
+    cell = {"type": "mlstm", "mlp": mlp, "mixer": {
+        "heads": z["heads"], "dim": z["nope"], "vdim": z["vdim"], "gate_cap": 15.0}}
+    return {"architecture": "Runidra",
+            "layers": [latent if i % 2 else cell for i in range(z["layers"])],
+            "norm": {"eps": 1e-5}, "streams": z["streams"], "logit_scale": 1.0,
+            "logit_softcap": 30.0, "vocab": z["vocab"], "width": z["width"]}
+
+
+def vurizen_like_config(z: dict) -> dict:
+    """vurizen_config with a recurrent and an attention layer in turn, every
+    attention layer with a cache of its own."""
+    cfg = vurizen_config(z)
+    cell, latent = cfg["layers"][0], cfg["layers"][1]
+    cfg["layers"] = [latent if i % 2 else cell for i in range(z["layers"])]
+    return cfg
+
+
 def design_compare(args) -> None:
     from parallax_amd.models.config import ModelConfig
     from parallax_amd.server.engine import Engine, EngineArgs
@@ -383,6 +428,10 @@ def design_compare(args) -> None:
             z = PUDIZEN_SIZES[size]
             pair = (("pudizen", pudizen_config(z)),
                     ("qwen3-like", qwen3_like_pudizen_config(z)))
+        elif args.design_pair == "runidra":
+            z = RUNIDRA_SIZES[size]
+            pair = (("runidra", runidra_config(z)),
+                    ("vurizen-like", vurizen_like_config(z)))
         else:
             z = DESIGN_SIZES[size]
             pair = (("vurizen", vurizen_config(z)),
@@ -491,21 +540,22 @@ def main():
                          "throughput of a Vurizen stack beside a DeepSeek-V3-"
                          "style stack of equal sizes (one GPU, random weights)")
     ap.add_argument("--design-pair", default="vurizen",
-                    choices=["vurizen", "sogidra", "zabusun", "pudizen"],
+                    choices=["vurizen", "sogidra", "zabusun", "pudizen", "runidra"],
                     help="which design --design-compare measures: vurizen "
                          "beside a DeepSeek-V3-style stack, sogidra beside "
                          "a Qwen3-style dense stack, zabusun beside a "
-                         "Qwen3-MoE-style stack, or pudizen beside a "
-                         "Qwen3-style dense stack")
+                         "Qwen3-MoE-style stack, pudizen beside a "
+                         "Qwen3-style dense stack, or runidra beside a "
+                         "vurizen stack")
     ap.add_argument("--design-sizes", default="s,m",
                     help="comma list of " + ",".join(DESIGN_SIZES)
-                    + " (the pudizen pair also has l)")
+                    + " (the pudizen and runidra pairs also have l)")
     ap.add_argument("--design-batch", type=int, default=8)
     ap.add_argument("--design-prompt", type=int, default=2048)
     ap.add_argument("--design-only", default="",
                     help="one design of the pair (vurizen | deepseek-like | "
                          "sogidra | qwen3-like | zabusun | qwen3-moe-like | "
-                         "pudizen; "
+                         "pudizen | runidra | vurizen-like; "
                          "default: both)")
     args = ap.parse_args()
     if args.design_compare:
