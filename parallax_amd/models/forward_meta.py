@@ -8,7 +8,7 @@ re-designed around our paged layout. All tensors live on the model's device.
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import TYPE_CHECKING, Optional
+from typing import TYPE_CHECKING, Dict, List, Optional, Tuple
 
 import torch
 
@@ -38,10 +38,15 @@ class ForwardMeta:
     # sequence's first token (filled for models that set `uses_prev_tokens`:
     # their embedding reads the pair)
     prev_ids: Optional[torch.Tensor] = None
+    # prefill only, host side: (first position, number of tokens) of every
+    # sequence's portion, for kernels whose workspace follows the context
+    # (None: unknown, such kernels are not used)
+    portions: Optional[List[Tuple[int, int]]] = None
     # derived per-token tables for packed-sequence kernels (built on first
     # use, shared by every layer of the forward)
     _token_seq: Optional[torch.Tensor] = None
     _query_bounds: Optional[torch.Tensor] = None
+    _contexts: Optional[Dict[int, tuple]] = None
 
     def token_seq(self) -> Optional[torch.Tensor]:
         """[T] int32: the batch row each packed token belongs to. None for a
@@ -65,6 +70,22 @@ class ForwardMeta:
                 torch.cumsum(self.query_lens, 0), (1, 0)
             ).to(torch.int32)
         return self._query_bounds
+
+    def window_contexts(self, window: int) -> Tuple[torch.Tensor, int]:
+        """The positions a sliding window lets the portions see, as dense
+        rows: sequence b's rows are plan[b] .. plan[b + 1] and start at
+        position plan[B + 1 + b]. Returns (plan [2 B + 1] int32, rows)."""
+        if self._contexts is None:
+            self._contexts = {}
+        if window not in self._contexts:
+            offs, los = [0], []
+            for start, count in self.portions:
+                lo = max(0, start - window + 1)
+                los.append(lo)
+                offs.append(offs[-1] + start + count - lo)
+            plan = torch.tensor(offs + los, dtype=torch.int32)
+            self._contexts[window] = (plan.to(self.positions.device), offs[-1])
+        return self._contexts[window]
 
     @property
     def num_tokens(self) -> int:

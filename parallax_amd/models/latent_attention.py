@@ -18,6 +18,12 @@ projection, RMS norm, up projection), the rotation may pair dimensions 2i and
 2i + 1, and the softmax may have a sink, a learned number per head whose
 exponential is one more term of the denominator. A layer that runs several
 times per token names the cache entry of the pass when it is called.
+
+Decode rows, short portions and float32 engines run absorbed. A bf16 portion
+that is long against the context it sees expands keys and values once instead
+(one GEMM over the context's latents) and attends on the matrix cores: a
+fraction of the operations, the same result up to the keys' and values'
+rounding to bf16.
 """
 
 from __future__ import annotations
@@ -36,6 +42,9 @@ from .rope import yarn_ramp_frequencies
 
 
 class LatentWindowAttention(nn.Module):
+    # a portion expands its context when that has at most so many rows a token
+    EXPAND_ROWS_PER_TOKEN = 16
+
     def __init__(self, hidden_size: int, heads: int, nope_dim: int, rot_width: int,
                  value_dim: int, rank: int, window: int, scale: float,
                  norm_eps: float, cache_layer_idx: int, owns_cache: bool,
@@ -77,6 +86,7 @@ class LatentWindowAttention(nn.Module):
         self.w_uv = nn.Parameter(torch.empty(heads, value_dim, rank), requires_grad=False)
         self.o_proj = RowParallelLinear(heads * value_dim, hidden_size)
         self._f32 = None  # (freq, w_uk, w_uv, sink), fp32, on the run device
+        self._w_kv = None  # [W_uk of all heads | W_uv of all heads]
 
     def _constants(self, device):
         if self._f32 is None or self._f32[0].device != device:
@@ -88,6 +98,27 @@ class LatentWindowAttention(nn.Module):
 
     def invalidate_constants(self) -> None:
         self._f32 = None
+        self._w_kv = None
+
+    def _expands(self, x: torch.Tensor, meta: ForwardMeta) -> bool:
+        if not (x.is_cuda and x.dtype == torch.bfloat16 and meta.is_prefill
+                and meta.portions and self.rank % 8 == 0
+                and ops.latent_expanded_supported(self.dn, self.dr, self.dv)):
+            return False
+        return meta.window_contexts(self.window)[1] \
+            <= self.EXPAND_ROWS_PER_TOKEN * x.shape[0]
+
+    def _attend_expanded(self, q, q_rot, cache, sink, meta: ForwardMeta):
+        H = self.heads
+        if self._w_kv is None or self._w_kv.device != q.device:
+            self._w_kv = torch.cat([self.w_uk.reshape(H * self.dn, self.rank),
+                                    self.w_uv.reshape(H * self.dv, self.rank)])
+        plan, rows = meta.window_contexts(self.window)
+        latent, k_rot = ops.latent_gather(cache, meta.block_tables, plan, rows,
+                                          self.rank)
+        return ops.latent_expanded_attention(
+            q, q_rot, ops.linear(latent, self._w_kv), k_rot, plan,
+            meta.query_bounds(), meta.positions, self.window, self.scale, sink)
 
     def forward(self, x: torch.Tensor, meta: ForwardMeta,
                 cache_layer_idx: Optional[int] = None) -> torch.Tensor:
@@ -110,6 +141,8 @@ class LatentWindowAttention(nn.Module):
         q_rot = ops.rope_rows(q, self.dn, self.dr, freq, self._mult,
                               self.rot_dims, meta.positions,
                               self.rot_interleaved)
+        if self._expands(x, meta):
+            return self.o_proj(self._attend_expanded(q, q_rot, cache, sink, meta))
         q_lat = torch.einsum("thd,hdr->thr", q[..., : self.dn].float(), w_uk)
         out_lat = ops.latent_window_attention(
             q_lat.contiguous(), q_rot, cache, meta.block_tables,

@@ -658,6 +658,9 @@ from .mix import (  # noqa: E402,F401
     group_rmsnorm_add,
     has_mix_extension,
     hyper_rmsnorm,
+    latent_expanded_attention,
+    latent_expanded_supported,
+    latent_gather,
     latent_kv_store,
     latent_window_attention,
     linear_f32,

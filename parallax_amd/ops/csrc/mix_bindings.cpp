@@ -42,6 +42,14 @@ void launch_softcap_logits(float*, const void*, float, float, int64_t, int,
 void launch_small_linear(float*, const void*, int64_t, const void*, int, int,
                          int, int64_t*, float*, const float*, int, int,
                          hipStream_t);
+void launch_latent_gather(void*, void*, const void*, const int*, int, const int*,
+                          int, int, int, int, int, hipStream_t);
+int latent_expanded_supported(int, int, int);
+void launch_latent_expanded_attention(void*, const void*, int64_t, const float*,
+                                      const void*, int64_t, const void*,
+                                      const int*, const int*, int, const int*,
+                                      int, int, int, int, int, int, float,
+                                      const float*, hipStream_t);
 void launch_mlstm(void*, float*, float*, float*, const void*, int64_t,
                   const void*, int64_t, const void*, int64_t, const void*,
                   int64_t, const float*, const float*, const void*, float,
@@ -1092,6 +1100,69 @@ void mlstm(torch::Tensor out, torch::Tensor q, torch::Tensor k, torch::Tensor v,
                cur_stream());
 }
 
+// lat [>= rows, rank], rot [>= rows, dr] bf16 from cache [blocks, block, rank +
+// dr] bf16; plan [2 B + 1] int32: row offsets [0 .. B], first positions [B]
+void latent_gather(torch::Tensor lat, torch::Tensor rot, torch::Tensor cache,
+                   torch::Tensor block_tables, torch::Tensor plan, int64_t rows) {
+  for (const torch::Tensor* t : {&lat, &rot, &cache})
+    TORCH_CHECK(t->is_cuda() && t->scalar_type() == at::kBFloat16 && t->is_contiguous());
+  TORCH_CHECK(lat.dim() == 2 && rot.dim() == 2 && cache.dim() == 3);
+  const int rank = lat.size(1), dr = rot.size(1);
+  TORCH_CHECK(cache.size(2) == rank + dr && rank % 8 == 0 && dr % 8 == 0);
+  TORCH_CHECK(lat.size(0) >= rows && rot.size(0) >= rows);
+  CHECK_I32(block_tables);
+  CHECK_I32(plan);
+  const int B = (plan.numel() - 1) / 2;
+  TORCH_CHECK(B >= 1 && plan.numel() == 2 * B + 1 && block_tables.dim() == 2 &&
+              block_tables.size(0) >= B);
+  launch_latent_gather(lat.data_ptr(), rot.data_ptr(), cache.data_ptr(),
+                       block_tables.data_ptr<int>(), (int)block_tables.stride(0),
+                       plan.data_ptr<int>(), B, (int)rows, (int)cache.size(1),
+                       rank, dr, cur_stream());
+}
+
+// out [T, H * dv] bf16, q [T, H, dn + dr] bf16 (token stride free), q_rot [T, H,
+// dr] fp32, kv [rows, H * (dn + dv)] bf16, k_rot [rows, dr] bf16, cu [B + 1]
+void latent_expanded_attention(torch::Tensor out, torch::Tensor q,
+                               torch::Tensor q_rot, torch::Tensor kv,
+                               torch::Tensor k_rot, torch::Tensor plan,
+                               torch::Tensor cu, torch::Tensor positions,
+                               int64_t window, double scale, torch::Tensor sink) {
+  for (const torch::Tensor* t : {&out, &q, &kv, &k_rot})
+    TORCH_CHECK(t->is_cuda() && t->scalar_type() == at::kBFloat16);
+  CHECK_F32C(q_rot);
+  TORCH_CHECK(q.dim() == 3 && q_rot.dim() == 3 && kv.dim() == 2 && k_rot.dim() == 2);
+  const int T = q.size(0), H = q.size(1), dr = q_rot.size(2);
+  const int dn = q.size(2) - dr;
+  const int dv = kv.size(1) / H - dn;
+  TORCH_CHECK(dn > 0 && dv > 0 && kv.size(1) == (int64_t)H * (dn + dv) &&
+              latent_expanded_supported(dn, dr, dv), "head widths");
+  TORCH_CHECK(q.stride(2) == 1 && q.stride(1) == dn + dr && q.stride(0) % 8 == 0 &&
+              ((uintptr_t)q.data_ptr() % 16) == 0, "query rows");
+  TORCH_CHECK(q_rot.size(0) == T && q_rot.size(1) == H);
+  TORCH_CHECK(kv.is_contiguous() && k_rot.is_contiguous() &&
+              k_rot.size(1) == dr && k_rot.size(0) >= kv.size(0));
+  TORCH_CHECK(out.is_contiguous() && out.dim() == 2 && out.size(0) == T &&
+              out.size(1) == (int64_t)H * dv);
+  CHECK_I32(plan);
+  CHECK_I32(cu);
+  CHECK_I32(positions);
+  const int B = cu.numel() - 1;
+  TORCH_CHECK(B >= 1 && plan.numel() == 2 * B + 1 && positions.numel() == T);
+  TORCH_CHECK(window >= 1 && window <= (1 << 30));
+  const bool has_sink = sink.numel() > 0;
+  if (has_sink) {
+    CHECK_F32C(sink);
+    TORCH_CHECK(sink.numel() == H);
+  }
+  launch_latent_expanded_attention(
+      out.data_ptr(), q.data_ptr(), q.stride(0), q_rot.data_ptr<float>(),
+      kv.data_ptr(), kv.stride(0), k_rot.data_ptr(), plan.data_ptr<int>(),
+      cu.data_ptr<int>(), B, positions.data_ptr<int>(), T / 128 + B, H, dn, dr, dv,
+      (int)window, (float)scale, has_sink ? sink.data_ptr<float>() : nullptr,
+      cur_stream());
+}
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("add_layernorm", &add_layernorm);
   m.def("latent_kv_store", &latent_kv_store);
@@ -1118,4 +1189,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("linear_f32", &linear_f32);
   m.def("route_softmax", &route_softmax);
   m.def("mlstm", &mlstm);
+  m.def("latent_gather", &latent_gather);
+  m.def("latent_expanded_attention", &latent_expanded_attention);
+  m.def("latent_expanded_supported", &latent_expanded_supported);
 }

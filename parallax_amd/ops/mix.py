@@ -133,6 +133,46 @@ def latent_window_attention(q_lat, q_rot, cache, block_tables, token_seq,
     return out
 
 
+def latent_expanded_supported(dn, dr, dv):
+    """Whether latent_expanded_attention tiles these head widths."""
+    return bool(_mix_ext().latent_expanded_supported(int(dn), int(dr), int(dv)))
+
+
+def latent_gather(cache, block_tables, plan, rows, rank):
+    """The `rows` context rows that ForwardMeta.window_contexts lists, out of
+    the paged latent cache, as (latents [.., rank], rotated parts [.., dr]).
+    On the GPU both are padded to a multiple of 256 rows (undefined content),
+    which keeps the shapes of the product that follows few."""
+    if not cache.is_cuda:
+        return ref.latent_gather(cache, block_tables, plan, rows, rank)
+    pad = (rows + 255) // 256 * 256
+    lat = torch.empty(pad, rank, dtype=cache.dtype, device=cache.device)
+    rot = torch.empty(pad, cache.shape[2] - rank, dtype=cache.dtype,
+                      device=cache.device)
+    _mix_ext().latent_gather(lat, rot, cache, block_tables, plan, int(rows))
+    return lat, rot
+
+
+def latent_expanded_attention(q, q_rot, kv, k_rot, plan, cu, positions, window,
+                              scale, sink=None):
+    """Sliding-window softmax attention of prompt portions over expanded keys
+    and values: q [T, H, dn + dr] bf16 (its first dn columns are used), q_rot
+    [T, H, dr] fp32, kv [rows, H * dn | H * dv] bf16 and k_rot [rows, dr] bf16
+    as window_contexts' plan lists them; cu [B + 1] int32 token bounds; sink
+    [H] fp32: one more term exp(sink[h]) of the denominator. Scores, softmax
+    and value sums are fp32. Returns [T, H * dv] bf16."""
+    if not q.is_cuda:
+        return ref.latent_expanded_attention(q, q_rot, kv, k_rot, plan, cu,
+                                             positions, window, scale, sink)
+    T, H, dr = q_rot.shape
+    out = torch.empty(T, kv.shape[1] - H * (q.shape[2] - dr), dtype=q.dtype,
+                      device=q.device)
+    _mix_ext().latent_expanded_attention(
+        out, q, q_rot, kv, k_rot, plan, cu, positions, int(window), float(scale),
+        sink if sink is not None else _empty(q_rot))
+    return out
+
+
 def gla_recurrence(q, k, v, z, z_bias, state, slots, cu, positions, inv_tau,
                    q_scale):
     """Gated-linear-attention recurrence over packed sequences; the fp32

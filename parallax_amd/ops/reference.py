@@ -644,6 +644,42 @@ def latent_window_attention(q_lat, q_rot, cache, block_tables, token_seq,
     return out
 
 
+def latent_gather(cache, block_tables, plan, rows, rank):
+    B = (plan.numel() - 1) // 2
+    p = plan.tolist()
+    bs, out = cache.shape[1], []
+    for b in range(B):
+        j = torch.arange(p[B + 1 + b], p[B + 1 + b] + p[b + 1] - p[b])
+        out.append(cache[block_tables[b].long()[j // bs], j % bs])
+    x = torch.cat(out)
+    return x[:, :rank].contiguous(), x[:, rank:].contiguous()
+
+
+def latent_expanded_attention(q, q_rot, kv, k_rot, plan, cu, positions, window,
+                              scale, sink=None):
+    T, H, dr = q_rot.shape
+    dn = q.shape[2] - dr
+    dv = kv.shape[1] // H - dn
+    B = cu.numel() - 1
+    p, c, pos = plan.tolist(), cu.tolist(), positions.tolist()
+    out = torch.empty(T, H, dv)
+    for b in range(B):
+        for t in range(c[b], c[b + 1]):
+            lo = max(0, pos[t] - window + 1)
+            r0 = p[b] + lo - p[B + 1 + b]
+            n = pos[t] - lo + 1
+            k = kv[r0:r0 + n, : H * dn].float().view(n, H, dn)
+            v = kv[r0:r0 + n, H * dn:].float().view(n, H, dv)
+            s = torch.einsum("hd,nhd->hn", q[t, :, :dn].float(), k) \
+                + q_rot[t] @ k_rot[r0:r0 + n].float().T
+            s = s * scale
+            if sink is not None:
+                s = torch.cat([s, sink.float().view(H, 1)], dim=-1)
+            w = torch.softmax(s, dim=-1)[:, :n]
+            out[t] = torch.einsum("hn,nhv->hv", w, v)
+    return out.view(T, H * dv).to(q.dtype)
+
+
 def gla_recurrence(q, k, v, z, z_bias, state, slots, cu, positions, inv_tau,
                    q_scale):
     T = q.shape[0]

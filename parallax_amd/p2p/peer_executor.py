@@ -477,6 +477,8 @@ class PeerExecutor:
             linear_cache=self.linear_cache,
             linear_slots=linear_slots,
             max_seq_len=max(seq_lens),
+            portions=[(s - n, n) for s, n in zip(seq_lens, qlens)]
+            if is_prefill and qlens else None,
         )
 
     def _send_forward(self, pkts: List[IntermediateRequest]) -> None:

@@ -818,6 +818,7 @@ class Engine:
             ) if self.linear_cache is not None else None,
             logits_indices=torch.tensor(logits_idx, dtype=torch.int64, device=dev),
             max_seq_len=max(seq_lens),
+            portions=[(c.start, c.num_tokens) for c in chunks],
             prev_ids=torch.tensor(prev_ids, dtype=torch.long, device=dev)
             if self.uses_prev_tokens else None,
         )

@@ -50,6 +50,7 @@ mix_sources = [
     os.path.join(CSRC, "mix_bindings.cpp"),
     os.path.join(CSRC, "layernorm.hip"),
     os.path.join(CSRC, "latent_attention.hip"),
+    os.path.join(CSRC, "latent_prefill.hip"),
     os.path.join(CSRC, "gla.hip"),
     os.path.join(CSRC, "sandwich_norm.hip"),
     os.path.join(CSRC, "row_attention.hip"),

@@ -272,3 +272,52 @@ def test_latent_window_attention_sink(dtype, H, rank, rot_w, window, ctx, decode
             None if seq is None else seq.to(DEV), pos.to(DEV), window, 0.1, ctx,
             None if sink is None else sink.to(DEV))
         torch.testing.assert_close(got.cpu(), want, rtol=1e-4, atol=1e-4)
+
+
+@pytest.mark.parametrize("H,dn,dr,dv,rank,window", [
+    (8, 64, 16, 48, 64, 96), (3, 24, 8, 72, 40, 33), (16, 128, 64, 128, 512, 1024),
+    (1, 8, 64, 8, 24, 1), (2, 104, 40, 120, 64, 500)])
+def test_latent_expanded_attention(H, dn, dr, dv, rank, window):
+    """Gathered contexts and tiled portions: sequences of unequal length, one
+    that starts inside its context, one of a single token, tiles that end
+    ragged; a planted key at the window's edge."""
+    from parallax_amd.models.forward_meta import ForwardMeta
+
+    bf = torch.bfloat16
+    portions = [(0, 300), (700, 150), (41, 1), (0, 2), (5, 128)]
+    bs, n_pages = 16, 400
+    cache = _rand(n_pages, bs, rank + dr, dtype=bf, seed=1)
+    perm = torch.randperm(n_pages, generator=torch.Generator().manual_seed(2)).int()
+    bt = perm[: 5 * 60].view(5, 60).contiguous()
+    pos = torch.cat([torch.arange(s, s + n) for s, n in portions]).int()
+    lens = torch.tensor([n for _, n in portions], dtype=torch.int32)
+    T = pos.numel()
+
+    def meta(dev):
+        return ForwardMeta(is_prefill=True, positions=pos.to(dev), slot_mapping=None,
+                           block_tables=bt.to(dev), seq_lens=None, query_lens=lens.to(dev),
+                           portions=portions)
+
+    mr, mg = meta("cpu"), meta(DEV)
+    plan, rows = mr.window_contexts(window)
+    assert rows == sum(s + n - max(0, s - window + 1) for s, n in portions)
+    lat_r, rot_r = ref.latent_gather(cache, bt, plan, rows, rank)
+    lat_g, rot_g = ops.latent_gather(cache.to(DEV), bt.to(DEV), mg.window_contexts(window)[0],
+                                     rows, rank)
+    assert torch.equal(lat_g[:rows].cpu(), lat_r) and torch.equal(rot_g[:rows].cpu(), rot_r)
+    kv = _rand(rows, H * (dn + dv), dtype=bf, seed=3)
+    q = _rand(T, H, dn + dr, dtype=bf, seed=4)
+    q_rot = _rand(T, H, dr, seed=5)
+    # one key of the second sequence stands out for every head: seen up to
+    # the window's edge and not beyond
+    kv[int(plan[1]) + min(20, window - 1), : H * dn] = 3.0
+    for sink in (None, _rand(H, seed=6), torch.full((H,), 5.0)):
+        want = ref.latent_expanded_attention(q.float(), q_rot, kv, rot_r, plan, mr.query_bounds(),
+                                             pos, window, 0.15, sink)
+        kv_pad = torch.full((rot_g.shape[0], kv.shape[1]), float("nan"), dtype=bf)
+        kv_pad[:rows] = kv
+        got = ops.latent_expanded_attention(
+            q.to(DEV), q_rot.to(DEV), kv_pad.to(DEV), rot_g, mg.window_contexts(window)[0],
+            mg.query_bounds(), pos.to(DEV), window, 0.15,
+            None if sink is None else sink.to(DEV))
+        _close(got, want, bf)
