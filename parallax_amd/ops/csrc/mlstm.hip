@@ -48,6 +48,28 @@ DEVINL void ml_load4<float>(const float* p, float* v) {
   v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
 }
 
+template <>
+DEVINL void ml_load4<bf16_t>(const bf16_t* p, float* v) {
+  const uint2 raw = *reinterpret_cast<const uint2*>(p);
+  v[0] = bf16_bits_to_f32((uint16_t)(raw.x & 0xffff));
+  v[1] = bf16_bits_to_f32((uint16_t)(raw.x >> 16));
+  v[2] = bf16_bits_to_f32((uint16_t)(raw.y & 0xffff));
+  v[3] = bf16_bits_to_f32((uint16_t)(raw.y >> 16));
+}
+template <typename T>
+DEVINL void ml_store4(T* p, const float* v);
+template <>
+DEVINL void ml_store4<float>(float* p, const float* v) {
+  *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+}
+template <>
+DEVINL void ml_store4<bf16_t>(bf16_t* p, const float* v) {
+  uint2 raw;
+  raw.x = (uint32_t)f32_to_bf16_bits(v[0]) | ((uint32_t)f32_to_bf16_bits(v[1]) << 16);
+  raw.y = (uint32_t)f32_to_bf16_bits(v[2]) | ((uint32_t)f32_to_bf16_bits(v[3]) << 16);
+  *reinterpret_cast<uint2*>(p) = raw;
+}
+
 // ---- decode ----------------------------------------------------------------------
 
 // grid (H, B); N = 4 (dv a multiple of 4) or 1 columns per thread.
@@ -627,36 +649,64 @@ __global__ __launch_bounds__(256, 2) void mlstm_chunk_kernel(
 
 // ---- head norm and output gate ---------------------------------------------------
 
-// one wave per (token, head)
-template <typename T>
+// lpr lanes per (token, head), 64 / lpr of those per wave. VEC: 4 consecutive
+// values per lane (dv a multiple of 4, at most 256; rows aligned), lpr a power of
+// two with 4 lpr >= dv; else lpr = 64 and a lane strides over the row.
+template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void mlstm_out_kernel(
     T* __restrict__ out, const float* __restrict__ o,
     const float* __restrict__ nq, const float* __restrict__ mm,
     const T* __restrict__ g, int64_t g_stride, const T* __restrict__ w,
     float eps, float* __restrict__ state, int64_t sw,
     const int64_t* __restrict__ slots, const int* __restrict__ cu, int B,
-    int rows, int H, int d, int dv) {
-  const int64_t row = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (row >= rows) return;
+    int64_t rows, int H, int d, int dv, int lpr) {
   const int lane = threadIdx.x & 63;
-  const int64_t t = row / H;
-  const int h = row % H;
-  const float m = mm[row];
-  const float den = 1.0f / (fmaxf(fabsf(nq[row]), expf(-m)) + ML_EPS);
-  const float* x = o + row * dv;
-  float ss = 0.f;
-  for (int i = lane; i < dv; i += 64) {
-    const float v = x[i] * den;
-    ss = fmaf(v, v, ss);
-  }
-  ss = wave_reduce_sum(ss);
-  const float r = den / sqrtf(ss / (float)dv + eps);
+  const int sub = lane % lpr;
+  const int64_t row = ((int64_t)blockIdx.x * 4 + (threadIdx.x >> 6)) * (64 / lpr) + lane / lpr;
+  const bool on = row < rows;     // all lanes stay for the reductions
+  const int64_t r_ = on ? row : rows - 1;
+  const int64_t t = r_ / H;
+  const int h = (int)(r_ % H);
+  const float m = mm[r_];
+  const float den = 1.0f / (fmaxf(fabsf(nq[r_]), expf(-m)) + ML_EPS);
+  const float* x = o + r_ * dv;
   const T* gr = g + t * g_stride + h * dv;
-  T* dst = out + row * dv;
-  for (int i = lane; i < dv; i += 64)
-    stf(dst + i, x[i] * r * ldf(w + h * dv + i) * ml_sigmoid(ldf(gr + i)));
+  T* dst = out + r_ * dv;
+  float v[4] = {0.f, 0.f, 0.f, 0.f};
+  float ss = 0.f;
+  if (VEC) {
+    const int i = sub * 4;
+    if (i < dv) ml_load4<float>(x + i, v);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      v[j] *= den;
+      ss = fmaf(v[j], v[j], ss);
+    }
+  } else {
+    for (int i = sub; i < dv; i += 64) {
+      const float z = x[i] * den;
+      ss = fmaf(z, z, ss);
+    }
+  }
+  for (int off = lpr >> 1; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
+  if (!on) return;
+  const float r = 1.0f / sqrtf(ss / (float)dv + eps);
+  if (VEC) {
+    const int i = sub * 4;
+    if (i < dv) {
+      float gv[4], wv[4];
+      ml_load4<T>(gr + i, gv);
+      ml_load4<T>(w + h * dv + i, wv);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] = v[j] * r * wv[j] * ml_sigmoid(gv[j]);
+      ml_store4<T>(dst + i, v);
+    }
+  } else {
+    for (int i = sub; i < dv; i += 64)
+      stf(dst + i, x[i] * (den * r) * ldf(w + h * dv + i) * ml_sigmoid(ldf(gr + i)));
+  }
   // a sequence's last token leaves its maximum in the state
-  for (int b = lane; b < B; b += 64) {
+  for (int b = sub; b < B; b += lpr) {
     const int e0 = cu ? cu[b] : b, e1 = cu ? cu[b + 1] : b + 1;
     if (e1 > e0 && e1 - 1 == t)
       state[(slots[b] * H + h) * sw + (int64_t)d * dv + d] = m;
@@ -711,10 +761,24 @@ static void launch_mlstm_t(void* out, float* o, float* nq, float* mm,
                        k_stride, (const T*)v, v_stride, gates, gate_bias, cap,
                        state, sw, slots, cu, positions, H, d, dv, G, TC, q_scale);
   }
-  hipLaunchKernelGGL((mlstm_out_kernel<T>), dim3((T_ * H + 3) / 4), dim3(256), 0,
-                     stream, (T*)out, o, nq, mm, (const T*)g, g_stride,
-                     (const T*)norm_w, eps, state, sw, slots, cu, B, T_ * H, H, d,
-                     dv);
+  const int64_t rows = (int64_t)T_ * H;
+  const int esz = sizeof(T);
+  const bool vec = dv % 4 == 0 && dv <= 256 && g_stride % 4 == 0 &&
+                   ((uintptr_t)g % (4 * esz)) == 0 &&
+                   ((uintptr_t)norm_w % (4 * esz)) == 0;
+  int lpr = 64;
+  if (vec)
+    while (lpr > 1 && lpr * 2 >= dv) lpr >>= 1;   // the smallest with 4 lpr >= dv
+  const int64_t per_block = 4 * (64 / lpr);
+#define MO_CALL(V)                                                             \
+  hipLaunchKernelGGL((mlstm_out_kernel<T, V>),                                 \
+                     dim3((rows + per_block - 1) / per_block), dim3(256), 0,   \
+                     stream, (T*)out, o, nq, mm, (const T*)g, g_stride,        \
+                     (const T*)norm_w, eps, state, sw, slots, cu, B, rows, H,  \
+                     d, dv, lpr)
+  if (vec) MO_CALL(true);
+  else MO_CALL(false);
+#undef MO_CALL
 }
 
 // path 0: one token per sequence (cu null); 1: token-serial; 2: chunks (bf16,

@@ -6,12 +6,13 @@
 //                   largest (lower index first among equals), weights = softmax
 //                   over those; rows E .. N are handed out as fp32 outputs.
 //
-// One workgroup takes 16 tokens and up to 16 NT columns. The 4 waves share out
-// the contraction (wave w takes every fourth block of 32) on the bf16 matrix
+// One workgroup takes 16 tokens and up to 16 NT columns. Its NW waves share out
+// the contraction (wave w takes every NW-th block of 32) on the bf16 matrix
 // cores with fp32 accumulators and add up through LDS, so a decode step of a
-// few tokens still has 4 x NT independent load streams in flight. For the
-// router the 16 rows of logits never leave LDS: a wave picks the experts of 4
-// tokens, one expert per round (a lane owns experts lane, lane + 64, ...).
+// few tokens still has NW x NT independent load streams in flight. For the
+// router the 16 rows of logits never leave LDS: a wave picks the experts of
+// 16 / NW tokens, one expert per round (a lane owns experts lane, lane + 64,
+// ...).
 #include "seq_common.h"
 
 #define SL_TOK 16
@@ -30,9 +31,9 @@ DEVINL bf16x8v sl_load8(const bf16_t* row, int k, int K) {
   return r;
 }
 
-// LDS: [4][16][NT * 16 + 1] partial sums; afterwards plane 0 holds the sums
-template <int NT, bool VEC, bool ROUTE>
-__global__ __launch_bounds__(256) void small_linear_kernel(
+// LDS: [NW][16][NT * 16 + 1] partial sums; afterwards plane 0 holds the sums
+template <int NT, int NW, bool VEC, bool ROUTE>
+__global__ __launch_bounds__(NW * 64) void small_linear_kernel(
     float* __restrict__ out, const bf16_t* __restrict__ x, int64_t x_stride,
     const bf16_t* __restrict__ w, int T_, int N, int K,
     int64_t* __restrict__ ids, float* __restrict__ wts,
@@ -46,8 +47,8 @@ __global__ __launch_bounds__(256) void small_linear_kernel(
   const bool tok_ok = t0 + l15 < T_;
   const bf16_t* xr = x + (int64_t)min(t0 + l15, T_ - 1) * x_stride;
   f32x4v acc[NT] = {};
-#pragma unroll 2
-  for (int k0 = wave * 32; k0 < K; k0 += 128) {
+#pragma unroll 4
+  for (int k0 = wave * 32; k0 < K; k0 += NW * 32) {
     const int k = k0 + l4 * 8;
     bf16x8v a = sl_load8<VEC>(xr, k, K);
     if (!tok_ok) a = bf16x8v{};
@@ -69,11 +70,11 @@ __global__ __launch_bounds__(256) void small_linear_kernel(
     for (int r = 0; r < 4; ++r)
       red[(wave * SL_TOK + l4 * 4 + r) * NP + i * 16 + l15] = acc[i][r];
   __syncthreads();
-  for (int idx = threadIdx.x; idx < SL_TOK * NT * 16; idx += 256) {
+  for (int idx = threadIdx.x; idx < SL_TOK * NT * 16; idx += NW * 64) {
     const int m = idx / (NT * 16), n = idx % (NT * 16);
     float v = red[m * NP + n];
 #pragma unroll
-    for (int wv = 1; wv < 4; ++wv) v += red[(wv * SL_TOK + m) * NP + n];
+    for (int wv = 1; wv < NW; ++wv) v += red[(wv * SL_TOK + m) * NP + n];
     const int t = t0 + m, col = n0 + n;
     if (ROUTE) {
       if (col < E && bias != nullptr) v += bias[col];
@@ -86,8 +87,8 @@ __global__ __launch_bounds__(256) void small_linear_kernel(
   if (!ROUTE) return;
   __syncthreads();
   constexpr int EC = (NT * 16 + 63) / 64;
-  for (int mm = 0; mm < 4; ++mm) {
-    const int m = wave * 4 + mm, t = t0 + m;
+  for (int mm = 0; mm < SL_TOK / NW; ++mm) {
+    const int m = wave * (SL_TOK / NW) + mm, t = t0 + m;
     if (t >= T_) break;
     float v[EC];
 #pragma unroll
@@ -139,10 +140,11 @@ static void launch_sl(float* out, const bf16_t* x, int64_t x_stride,
                       float* wts, const float* bias, int E, int top, bool vec,
                       hipStream_t stream) {
   const dim3 grid((T_ + SL_TOK - 1) / SL_TOK, (N + NT * 16 - 1) / (NT * 16));
-  const size_t shm = sizeof(float) * 4 * SL_TOK * (NT * 16 + 1);
+  constexpr int NW = NT <= 4 ? 8 : 4;   // partial sums within 64 KB of LDS
+  const size_t shm = sizeof(float) * NW * SL_TOK * (NT * 16 + 1);
 #define SL_CALL(V, R)                                                         \
-  hipLaunchKernelGGL((small_linear_kernel<NT, V, R>), grid, dim3(256), shm,   \
-                     stream, out, x, x_stride, w, T_, N, K, ids, wts, bias, E, \
+  hipLaunchKernelGGL((small_linear_kernel<NT, NW, V, R>), grid, dim3(NW * 64), \
+                     shm, stream, out, x, x_stride, w, T_, N, K, ids, wts, bias, E, \
                      top)
   if (ids != nullptr) {
     if (vec) SL_CALL(true, true);
