@@ -21,3 +21,4 @@ from . import sogidra  # noqa: F401
 from . import zabusun  # noqa: F401
 from . import pudizen  # noqa: F401
 from . import runidra  # noqa: F401
+from . import domelix  # noqa: F401

@@ -21,6 +21,14 @@ _PLAIN_ROW_DESIGNS = ("Pudizen",)
 # ('loop') over several copies of the residual stream ('streams')
 _LOOPED_DESIGNS = ("Runidra",)
 
+# layer-list designs whose layers run a mixer and a feed-forward side by side
+# on two norms of the same stream, with matrix-state mixers and a 'parallel'
+# type whose recurrent half keeps a matrix per head
+_TWO_NORM_DESIGNS = ("Domelix",)
+
+# layer types that keep recurrent state in a per-request slot
+_STATE_TYPES = ("gla", "parallel", "mlstm", "retention", "delta")
+
 
 def feed_forward_kind(mlp: Dict[str, Any]) -> str:
     """'moe' or 'dense' of a layer-list feed-forward entry: its 'kind', or by
@@ -107,9 +115,10 @@ class ModelConfig:
     linear_value_head_dim: int = 0
     linear_conv_kernel_dim: int = 4
 
-    # -- per-layer stacks (vurizen, sogidra, zabusun, pudizen, runidra): every layer carries its own mixer and
-    # feed-forward description; the flat fields above hold the first layer's
-    # values only so that sizing helpers have something to read ----------------
+    # -- per-layer stacks (vurizen, sogidra, zabusun, pudizen, runidra, domelix):
+    # every layer carries its own mixer and feed-forward description; the flat
+    # fields above hold the first layer's values only so that sizing helpers
+    # have something to read -------------------------------------------------
     layer_specs: Optional[List[Dict[str, Any]]] = None
     # stacks that run some layers several times: entry i is a layer RUN (with a
     # cache entry or state of its own) and layer_weights[i] the index of the
@@ -213,8 +222,20 @@ class ModelConfig:
                 if sp["type"] == "gla":
                     shapes.append(((0,), (int(mx["heads"]), int(mx["dim"]),
                                           int(mx["vdim"]))))
-                elif sp["type"] == "parallel":   # the recurrent half: a vector
+                elif sp["type"] == "parallel" and "width" in mx["right"]:
+                    # the recurrent half keeps a vector
                     shapes.append(((0,), (int(mx["right"]["width"]),)))
+                elif sp["type"] in ("retention", "delta", "parallel"):
+                    # one [key width, value width] matrix per head; the delta
+                    # rule also keeps its convolution's last taps - 1 inputs
+                    m = mx["right"] if sp["type"] == "parallel" else mx
+                    H, d = int(m["heads"]), int(m["dim"])
+                    dv = int(m.get("vdim", d))
+                    conv = (0,)
+                    if sp["type"] == "delta":
+                        conv = (2 * int(m.get("kv_heads", H)) * d + H * dv,
+                                int(m["conv"]) - 1)
+                    shapes.append((conv, (H, d, dv)))
                 elif sp["type"] == "mlstm":      # matrix, normaliser, maximum
                     shapes.append(((0,), (int(mx["heads"]), mlstm_state_width(
                         int(mx["dim"]), int(mx["vdim"])))))
@@ -242,7 +263,7 @@ class ModelConfig:
         """Whether any layer keeps recurrent state in a per-request slot."""
         if self.layer_specs is not None:
             return self.architecture not in _PLAIN_ROW_DESIGNS and any(
-                sp["type"] in ("gla", "parallel", "mlstm") for sp in self.layer_specs)
+                sp["type"] in _STATE_TYPES for sp in self.layer_specs)
         return bool(self.layer_types) and "linear_attention" in self.layer_types
 
     def layer_type(self, layer_idx: int) -> str:
@@ -281,11 +302,15 @@ class ModelConfig:
         and 'norm' {"eps", "groups"}. Runidra has 'mlstm' and a
         'latent_attention' with a query latent and sinks, and the top-level
         keys 'streams', 'loop' {"start", "stop", "times"}, 'logit_scale' and
-        'logit_softcap'."""
+        'logit_softcap'. Domelix has 'parallel' (softmax attention with a
+        distance bias beside lightning attention), 'delta' (gated delta rule)
+        and 'retention'."""
         if cfg["architecture"] in _PLAIN_ROW_DESIGNS:
             return cls._from_plain_row_config(cfg)
         if cfg["architecture"] in _LOOPED_DESIGNS:
             return cls._from_looped_config(cfg)
+        if cfg["architecture"] in _TWO_NORM_DESIGNS:
+            return cls._from_two_norm_config(cfg)
         layers = cfg["layers"]
         kinds = {"gla": "linear_attention", "latent_attention": "latent_attention",
                  "attention": "diff_attention",
@@ -477,6 +502,60 @@ class ModelConfig:
                 mc.shared_expert_intermediate_size = int(moes[0]["shared"]["ff"])
             if not dense:
                 mc.intermediate_size = mc.moe_intermediate_size
+        return mc
+
+    @classmethod
+    def _from_two_norm_config(cls, cfg: Dict[str, Any]) -> "ModelConfig":
+        """Layers of 'parallel', 'delta' and 'retention' mixers, each beside
+        routed experts (or nothing): see models/domelix.py."""
+        layers = cfg["layers"]
+        kinds = {"parallel": "parallel_attention_recurrent",
+                 "delta": "linear_attention", "retention": "linear_attention"}
+        for sp in layers:
+            if sp["type"] not in kinds:
+                raise ValueError(f"unknown layer type {sp['type']!r}")
+            mlp = sp.get("mlp")
+            if mlp is not None and feed_forward_kind(mlp) != "moe":
+                raise ValueError(f"unknown feed-forward kind {mlp.get('kind')!r}")
+        first = layers[0]["mixer"]
+        first = first.get("left", first)
+        mc = cls(
+            architecture=cfg["architecture"],
+            model_type=str(cfg["architecture"]).lower(),
+            vocab_size=int(cfg["vocab"]),
+            hidden_size=int(cfg["width"]),
+            num_layers=len(layers),
+            num_heads=int(first["heads"]),
+            num_kv_heads=int(first.get("kv_heads", first["heads"])),
+            head_dim=int(first["dim"]),
+            rms_norm_eps=float(cfg["norm"]["eps"]),
+            max_position_embeddings=int(cfg.get("max_positions", 1 << 20)),
+            layer_types=[kinds[sp["type"]] for sp in layers],
+            eos_token_ids=[],
+            bos_token_id=None,
+            torch_dtype=cfg.get("torch_dtype", "bfloat16"),
+            layer_specs=layers,
+            raw=cfg,
+        )
+        # the flat fields of the recurrent layers: the delta rule's sizes if
+        # there is one, else any other's
+        states = [sp["mixer"].get("right", sp["mixer"])
+                  for sp in sorted(layers, key=lambda sp: sp["type"] != "delta")]
+        m = states[0]
+        mc.linear_num_value_heads = int(m["heads"])
+        mc.linear_num_key_heads = int(m.get("kv_heads", m["heads"]))
+        mc.linear_key_head_dim = int(m["dim"])
+        mc.linear_value_head_dim = int(m.get("vdim", m["dim"]))
+        mc.linear_conv_kernel_dim = int(m.get("conv", 1))
+        moes = [sp["mlp"] for sp in layers if sp.get("mlp") is not None]
+        if moes:
+            r = moes[0]["router"]
+            g = r.get("groups") or {}
+            mc.num_experts = int(r["experts"])
+            mc.num_experts_per_tok = int(r["top"])
+            mc.moe_intermediate_size = int(moes[0]["expert"]["ff"])
+            mc.intermediate_size = mc.moe_intermediate_size
+            mc.n_group, mc.topk_group = int(g.get("count", 1)), int(g.get("keep", 1))
         return mc
 
     @classmethod

@@ -47,6 +47,7 @@ class ForwardMeta:
     _token_seq: Optional[torch.Tensor] = None
     _query_bounds: Optional[torch.Tensor] = None
     _contexts: Optional[Dict[int, tuple]] = None
+    _rope_tables: Optional[Dict[tuple, torch.Tensor]] = None
 
     def token_seq(self) -> Optional[torch.Tensor]:
         """[T] int32: the batch row each packed token belongs to. None for a
@@ -86,6 +87,17 @@ class ForwardMeta:
             plan = torch.tensor(offs + los, dtype=torch.int32)
             self._contexts[window] = (plan.to(self.positions.device), offs[-1])
         return self._contexts[window]
+
+    def rope_table(self, key: tuple, freq: torch.Tensor) -> torch.Tensor:
+        """The tokens' (cos, sin) pairs at frequencies `freq`, [T, 2 n] fp32;
+        layers whose rotations have the same `key` share one table."""
+        if self._rope_tables is None:
+            self._rope_tables = {}
+        if key not in self._rope_tables:
+            from .. import ops
+
+            self._rope_tables[key] = ops.rope_table(self.positions, freq)
+        return self._rope_tables[key]
 
     @property
     def num_tokens(self) -> int:

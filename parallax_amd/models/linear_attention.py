@@ -1,6 +1,8 @@
 """Recurrent sequence mixers whose state lives in the engine's per-request
-slots: gated linear attention (below), minGRU (class MinGRU) and the matrix
-LSTM (class MLSTM).
+slots: gated linear attention (below), minGRU (class MinGRU), the matrix LSTM
+(class MLSTM), linear attention with a fixed decay per head (class
+DecayLinearAttention: retention, lightning attention) and the gated delta rule
+(class GatedDeltaRule).
 
 Gated linear attention (GLA): a matrix-valued recurrent state per head with
 a data-dependent decay per key channel,
@@ -18,6 +20,8 @@ activation dtype.
 """
 
 from __future__ import annotations
+
+from typing import Sequence
 
 import torch
 import torch.nn as nn
@@ -176,3 +180,151 @@ class MLSTM(nn.Module):
                       meta.linear_slots, meta.query_bounds(), meta.positions,
                       x.dtype)
         return self.o_proj(o)
+
+
+class DecayLinearAttention(nn.Module):
+    """Linear attention with one fixed decay per head, no softmax and no
+    denominator,
+
+        S_t = decay_h S_(t-1) + k_t v_t^T,     o_t = S_t^T q_t,
+
+    S [dim, vdim] from zero, then a norm, an output gate and the output
+    projection. Switches make it retention (q and k rotated by position on
+    their first rot_dims dimensions, pairs i, i + rot_dims / 2; k times
+    k_scale; each head's o divided by its RMS; silu gate) or lightning
+    attention (silu on q, k and v; the heads normed together with a weight,
+    `norm_all`; sigmoid gate). Angles, decays, state, norm and gate are fp32
+    (ops.decay_attention, ops.gated_rmsnorm); the state lives in
+    LinearStateCache slots.
+
+    own_proj False: a caller merges the input projections [q | k | v | g]
+    (`proj_sizes`) with others of the same input and hands their columns to
+    mix()."""
+
+    def __init__(self, hidden_size: int, heads: int, dim: int, vdim: int,
+                 decay: Sequence[float], norm_eps: float, state_layer_idx: int, *,
+                 silu: bool = False, rot_dims: int = 0, rot_base: float = 10000.0,
+                 k_scale: float = 1.0, norm_all: bool = False,
+                 gate_act: str = "silu", own_proj: bool = True):
+        super().__init__()
+        if len(decay) != heads:
+            raise ValueError(f"{len(decay)} decays for {heads} heads")
+        if rot_dims % 2 or rot_dims > dim:
+            raise ValueError(f"cannot rotate {rot_dims} of {dim} dimensions")
+        self.heads, self.dim, self.vdim = heads, dim, vdim
+        self.eps = norm_eps
+        self.state_layer_idx = state_layer_idx
+        self.silu, self.k_scale = bool(silu), float(k_scale)
+        self.norm_all, self.gate_act = bool(norm_all), gate_act
+        self._powers = ops.decay_powers(decay)
+        self._rot_key = (int(rot_dims), float(rot_base))
+        self._freq = None
+        if rot_dims:
+            i = torch.arange(0, rot_dims, 2, dtype=torch.float64)
+            self._freq = (float(rot_base) ** (-i / rot_dims)).float()
+        self.proj_sizes = [heads * dim, heads * dim, heads * vdim, heads * vdim]
+        self.in_proj = MergedColumnParallelLinear(hidden_size, self.proj_sizes) \
+            if own_proj else None
+        self.norm_weight = nn.Parameter(torch.empty(heads * vdim),
+                                        requires_grad=False) if norm_all else None
+        self.o_proj = RowParallelLinear(heads * vdim, hidden_size)
+
+    def invalidate_constants(self) -> None:
+        pass
+
+    def mix(self, qkvg: torch.Tensor, meta: ForwardMeta) -> torch.Tensor:
+        """qkvg: the projections' columns (a strided view is fine) -> [T, heads
+        * vdim]."""
+        T, H = qkvg.shape[0], self.heads
+        q, k, v, g = torch.split(qkvg, self.proj_sizes, dim=-1)
+        dev = qkvg.device
+        if self._powers.device != dev:
+            self._powers = self._powers.to(dev)
+            self._freq = self._freq.to(dev) if self._freq is not None else None
+        cs = meta.rope_table(self._rot_key, self._freq) \
+            if self._freq is not None else None
+        o = ops.decay_attention(
+            q.view(T, H, self.dim), k.view(T, H, self.dim), v.view(T, H, self.vdim),
+            self._powers, self.k_scale, self.silu, cs,
+            meta.linear_cache.recurrent_states[self.state_layer_idx],
+            meta.linear_slots, meta.query_bounds(), meta.positions)
+        return ops.gated_rmsnorm(o, g, self.norm_weight, self.eps,
+                                 self.o_proj.weight.dtype, whole=self.norm_all,
+                                 act=self.gate_act)
+
+    def forward(self, x: torch.Tensor, meta: ForwardMeta) -> torch.Tensor:
+        return self.o_proj(self.mix(self.in_proj(x), meta))
+
+
+class GatedDeltaRule(nn.Module):
+    """Gated delta rule: `kv_heads` query/key heads of width dim, `heads` value
+    heads of width vdim (head h reads q/k head h // (heads / kv_heads)). q, k
+    and v pass a causal depthwise convolution over time and silu; q and k
+    become unit vectors, q times dim^-1/2; beta = sigmoid(W_b h), g =
+    exp(-exp(A_log) softplus(W_a h + dt_bias)), one each per head:
+
+        S <- g S,   u = beta (v - S^T k),   S <- S + k u^T,   o = S^T q;
+
+    each head's o is divided by its RMS, times a weight shared by the heads,
+    times silu(W_g h), then the output projection. Unit norms, gates, decays,
+    state and the head norm are fp32; so are the gates' pre-activations
+    (ops.linear_f32), which end in exponentials. The state and the
+    convolution's last inputs live in LinearStateCache slots."""
+
+    def __init__(self, hidden_size: int, heads: int, kv_heads: int, dim: int,
+                 vdim: int, taps: int, norm_eps: float, state_layer_idx: int):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError(f"{heads} heads do not divide into {kv_heads} "
+                             "query/key heads")
+        if taps < 1:
+            raise ValueError("a convolution has at least one tap")
+        self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
+        self.eps = norm_eps
+        self.state_layer_idx = state_layer_idx
+        self.conv_sizes = [kv_heads * dim, kv_heads * dim, heads * vdim]
+        self.conv_width = sum(self.conv_sizes)
+        # one GEMM for q | k | v | output gate
+        self.in_proj = MergedColumnParallelLinear(
+            hidden_size, self.conv_sizes + [heads * vdim])
+        self.conv_weight = nn.Parameter(torch.empty(self.conv_width, taps),
+                                        requires_grad=False)
+        # step sizes, then decays
+        self.gate_weight = nn.Parameter(torch.empty(2 * heads, hidden_size),
+                                        requires_grad=False)
+        self.a_log = nn.Parameter(torch.empty(heads), requires_grad=False)
+        self.dt_bias = nn.Parameter(torch.empty(heads), requires_grad=False)
+        self.norm_weight = nn.Parameter(torch.empty(vdim), requires_grad=False)
+        self.o_proj = RowParallelLinear(heads * vdim, hidden_size)
+        self._f32 = None
+
+    def load_conv(self, which: int, t: torch.Tensor) -> None:
+        """which: 0 = q, 1 = k, 2 = v; t [channels, taps]."""
+        off = sum(self.conv_sizes[:which])
+        self.conv_weight.data[off : off + self.conv_sizes[which]].copy_(t)
+
+    def load_gate(self, which: int, t: torch.Tensor) -> None:
+        """which: 0 = step size, 1 = decay."""
+        self.gate_weight.data[which * self.heads : (which + 1) * self.heads].copy_(t)
+
+    def invalidate_constants(self) -> None:
+        self._f32 = None
+
+    def forward(self, x: torch.Tensor, meta: ForwardMeta) -> torch.Tensor:
+        if self._f32 is None or self._f32[0].device != x.device:
+            self._f32 = tuple(p.detach().float().contiguous().to(x.device)
+                              for p in (self.a_log, self.dt_bias))
+        T, cache, idx = x.shape[0], meta.linear_cache, self.state_layer_idx
+        y = self.in_proj(x)
+        cu = meta.query_bounds()
+        mixed = ops.short_conv(y[:, : self.conv_width], self.conv_weight,
+                               cache.conv_states[idx], meta.linear_slots, cu,
+                               meta.positions, x.dtype)
+        q, k, v = torch.split(mixed, self.conv_sizes, dim=-1)
+        o = ops.gated_delta_rule(
+            q.view(T, self.kv_heads, self.dim), k.view(T, self.kv_heads, self.dim),
+            v.view(T, self.heads, self.vdim), ops.linear_f32(x, self.gate_weight),
+            *self._f32, cache.recurrent_states[idx], meta.linear_slots, cu,
+            meta.positions)
+        return self.o_proj(ops.gated_rmsnorm(o, y[:, self.conv_width :],
+                                             self.norm_weight, self.eps, x.dtype))

@@ -28,16 +28,27 @@ class MoERouter(nn.Module):
     logit_bias: softmax scoring adds a learned number per expert to its logit
     (before the choice). extra_rows: further rows of the same weight that are
     no experts (a shared expert's gate, say); route() returns their fp32
-    outputs beside the routing. Both want softmax scoring with weights
-    normalised over the chosen experts and run in one kernel (ops.route_softmax)."""
+    outputs beside the routing. fused: softmax scoring, limited to the best
+    topk_group of n_group runs of neighbouring experts (a run is as good as its
+    best expert). All three want weights normalised over the chosen experts
+    and run in one kernel (ops.route_softmax)."""
 
     def __init__(self, cfg: ModelConfig, logit_bias: bool = False,
-                 extra_rows: int = 0):
+                 extra_rows: int = 0, fused: bool = False):
         super().__init__()
-        self.fused = logit_bias or extra_rows > 0
-        if self.fused and (cfg.scoring_func != "softmax" or not cfg.norm_topk_prob):
-            raise ValueError("logit bias and extra rows come with softmax "
-                             "weights over the chosen experts")
+        self.fused = fused or logit_bias or extra_rows > 0
+        if self.fused:
+            if cfg.scoring_func != "softmax" or not cfg.norm_topk_prob:
+                raise ValueError("the one-kernel router has softmax weights over "
+                                 "the chosen experts")
+            groups = max(1, cfg.n_group)
+            if cfg.num_experts % groups or not 1 <= cfg.topk_group <= groups \
+                    or cfg.num_experts_per_tok > \
+                    cfg.num_experts // groups * cfg.topk_group:
+                raise ValueError(
+                    f"cannot choose {cfg.num_experts_per_tok} of "
+                    f"{cfg.num_experts} experts in {cfg.topk_group} of {groups} "
+                    "groups")
         self.num_experts = cfg.num_experts
         self.top_k = cfg.num_experts_per_tok
         self.norm_topk_prob = cfg.norm_topk_prob
@@ -68,7 +79,7 @@ class MoERouter(nn.Module):
                 self._b32 is None or self._b32.device != x.device):
             self._b32 = self.logit_bias.detach().float().contiguous()
         return ops.route_softmax(x, self.weight, self._b32, self.num_experts,
-                                 self.top_k)
+                                 self.top_k, self.n_group, self.topk_group)
 
     def forward(self, x: torch.Tensor):
         """x: [T, H] -> (topk_ids [T, k] long, topk_weights [T, k] float)."""

@@ -6,7 +6,7 @@ depend on how its prompt was cut or batched. Queries are prepared in fp32 by
 ops.qkv_store, which also scatters the step's keys and values; scores,
 softmax and the per-head post-processing are fp32.
 
-Four mixers are built on it:
+Five mixers are built on it:
 
 DifferentialAttention — every head has TWO query/key maps over the same
 values. With a1, a2 the two softmax results, o = a1 - lambda * a2, then o is
@@ -42,12 +42,19 @@ optionally rotated values: the value of position j is turned by j over its
 whole width before it is cached, and a head's result at position i is turned
 back by i, so that the result depends on i - j only.
 
+DistanceBiasAttention — no rotation: a learned number per head and distance
+bucket is added to the scaled score (bucket n for small distances n, then
+logarithmic up to a largest distance); full causal mask; the softmax's
+denominator also holds exp(sink_h); the concatenated heads are multiplied
+element by element with sigmoid(W_g h).
+
 Any of them may read ANOTHER layer's cache rows (`owns_cache=False`) with
 its own queries. All sizes and constants are constructor arguments.
 """
 
 from __future__ import annotations
 
+import functools
 import math
 from typing import Optional
 
@@ -59,6 +66,25 @@ from ..parallel.comm import get_comm
 from ..parallel.layers import MergedColumnParallelLinear, RowParallelLinear
 from .forward_meta import ForwardMeta
 from .rope import yarn_ramp_frequencies
+
+
+@functools.lru_cache(maxsize=64)
+def distance_buckets(buckets: int, limit: int) -> torch.Tensor:
+    """Bucket of every distance 0 .. limit (int64; farther ones share the last
+    entry): n itself below h = buckets // 2, then min(buckets - 1, h +
+    floor(ln(n / h) / ln(limit / h) * (buckets - h))). The floor is decided in
+    whole numbers: its value is at least m where n^K h^m >= limit^m h^K, K =
+    buckets - h."""
+    h = buckets // 2
+    K = buckets - h
+    if h < 1 or limit <= h:
+        raise ValueError(f"{buckets} distance buckets cannot reach up to {limit}")
+    out, m = list(range(min(h, limit + 1))), 0
+    for n in range(h, limit + 1):
+        while m < K and n ** K * h ** (m + 1) >= limit ** (m + 1) * h ** K:
+            m += 1
+        out.append(min(buckets - 1, h + m))
+    return torch.tensor(out, dtype=torch.int64)
 
 
 class _RowAttentionBase(nn.Module):
@@ -324,6 +350,61 @@ class RotaryRowAttention(_RowAttentionBase):
             max_seq_len=meta.max_seq_len, query_bounds=meta.query_bounds(),
             head_bias=bias, out_rot_cs=v_cs,
             out_rot_interleaved=self.rot_interleaved,
+        )
+
+    def forward(self, x: torch.Tensor, meta: ForwardMeta) -> torch.Tensor:
+        parts = self.in_proj.split_output(self.in_proj(x))
+        return self.o_proj(self.mix(parts, meta, x.dtype))
+
+
+class DistanceBiasAttention(_RowAttentionBase):
+    maps = 1
+
+    def __init__(self, hidden_size: int, heads: int, kv_heads: int, dim: int,
+                 value_dim: int, scale: float, bias_max: int, norm_eps: float,
+                 cache_layer_idx: int, owns_cache: bool = True, *,
+                 buckets: int = 32, own_proj: bool = True):
+        super().__init__(hidden_size, heads, kv_heads, dim, value_dim, scale,
+                         norm_eps, cache_layer_idx, owns_cache, False, True,
+                         extra_sizes=[heads * value_dim], own_proj=own_proj)
+        self.bias_max = int(bias_max)
+        self.rel = nn.Parameter(torch.empty(buckets, heads), requires_grad=False)
+        self.sink = nn.Parameter(torch.empty(heads), requires_grad=False)
+        self._f32 = None
+
+    def load_rel(self, t: torch.Tensor) -> None:
+        """The table's rows (distance buckets) follow the checkpoint's tensor."""
+        self.rel = nn.Parameter(
+            t.to(dtype=self.rel.dtype, device=self.rel.device).clone(),
+            requires_grad=False)
+
+    def invalidate_constants(self) -> None:
+        self._f32 = None
+
+    def _constants(self, device):
+        if self._f32 is None or self._f32[0].device != device:
+            idx = distance_buckets(self.rel.shape[0], self.bias_max)
+            rel = self.rel.detach().float().cpu()[idx]       # [bias_max + 1, heads]
+            self._f32 = (rel.t().contiguous().to(device),
+                         self.sink.detach().float().contiguous().to(device))
+        return self._f32
+
+    def mix(self, parts, meta: ForwardMeta, out_dtype) -> torch.Tensor:
+        """parts: the projections [q, (k, v,) gate pre-activations] of the
+        step's tokens (strided views are fine) -> [T, heads * value_dim]."""
+        q, gate = parts[0], parts[-1]
+        k, v = (parts[1], parts[2]) if self.owns_cache else (None, None)
+        bias, sink = self._constants(q.device)
+        cache = meta.mla_cache.layer(self.cache_layer_idx)
+        q32 = ops.qkv_store(q, k, v, meta.positions, meta.slot_mapping, cache,
+                            self.dim, None, 0.0, 0)
+        return ops.row_attention(
+            q32, cache, None, meta.block_tables, meta.token_seq(),
+            meta.positions, self.heads, self.kv_heads, 1, self.dim, self.vdim,
+            0, 0, self.scale, 0.0, 0.0, None, 1.0, out_dtype,
+            max_seq_len=meta.max_seq_len, query_bounds=meta.query_bounds(),
+            gate=gate, dist_bias=bias, sink=sink,
+            bf16_queries=q.dtype == torch.bfloat16,
         )
 
     def forward(self, x: torch.Tensor, meta: ForwardMeta) -> torch.Tensor:

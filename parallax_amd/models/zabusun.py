@@ -46,38 +46,9 @@ from .config import ModelConfig
 from .forward_meta import ForwardMeta
 from .linear_attention import MinGRU
 from .moe import FusedMoE
+from .parallel_mixer import ParallelMixer
 from .registry import register_model
 from .row_attention import GatedSigmoidAttention
-
-
-class ParallelMixer(nn.Module):
-    """Two mixers over the same input: out = left_scale * left(h) +
-    right_scale * right(h). The input projections of both are one GEMM; the
-    two results stay apart (forward returns both) so that the caller's
-    residual kernel scales and adds them in fp32."""
-
-    def __init__(self, hidden_size: int, left: nn.Module, right: nn.Module,
-                 left_scale: float, right_scale: float):
-        super().__init__()
-        self.left, self.right = left, right
-        self.left_scale, self.right_scale = float(left_scale), float(right_scale)
-        self.n_left = len(left.proj_sizes)
-        self.in_proj = MergedColumnParallelLinear(
-            hidden_size, list(left.proj_sizes) + list(right.proj_sizes))
-        self._right_width = sum(right.proj_sizes)
-
-    def invalidate_constants(self) -> None:
-        self.left.invalidate_constants()
-        self.right.invalidate_constants()
-
-    def forward(self, h: torch.Tensor, meta: ForwardMeta):
-        y = self.in_proj(h)
-        parts = self.in_proj.split_output(y)
-        a = self.left.o_proj(self.left.mix(parts[: self.n_left], meta, h.dtype))
-        # the right mixer's pre-activations are adjacent columns of y
-        b = self.right.o_proj(
-            self.right.mix(y[:, y.shape[1] - self._right_width:], meta))
-        return a, b
 
 
 class ClampedGluMLP(nn.Module):

@@ -652,7 +652,10 @@ from .mix import (  # noqa: E402,F401
     biased_glu,
     branch_rmsnorm_add,
     clamped_glu,
+    decay_attention,
+    decay_powers,
     embed_streams,
+    gated_delta_rule,
     gated_rmsnorm,
     gla_recurrence,
     group_rmsnorm_add,
@@ -667,14 +670,17 @@ from .mix import (  # noqa: E402,F401
     mingru_scan,
     mlstm,
     pair_hash_embedding,
+    parallel_rmsnorm_add,
     pool_cache_update,
     qkv_store,
     relu_squared,
     rope_rows,
+    rope_table,
     rotate_heads,
     route_softmax,
     row_attention,
     sandwich_rmsnorm,
+    short_conv,
     softcap_logits,
     xielu,
 )

@@ -110,29 +110,131 @@ __global__ __launch_bounds__(256) void gla_recurrence_kernel(
   }
 }
 
-// out[t, h*dv + j] = o[t,h,j] / rms(o[t,h,:]) * w[j] * silu(gate[t, h*dv + j])
-// one wave per (token, head)
 template <typename T>
+DEVINL void gn4_load(const T* p, float* v);
+template <>
+DEVINL void gn4_load<float>(const float* p, float* v) {
+  const float4 a = *reinterpret_cast<const float4*>(p);
+  v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
+}
+template <>
+DEVINL void gn4_load<bf16_t>(const bf16_t* p, float* v) {
+  const uint2 raw = *reinterpret_cast<const uint2*>(p);
+  v[0] = bf16_bits_to_f32((uint16_t)(raw.x & 0xffff));
+  v[1] = bf16_bits_to_f32((uint16_t)(raw.x >> 16));
+  v[2] = bf16_bits_to_f32((uint16_t)(raw.y & 0xffff));
+  v[3] = bf16_bits_to_f32((uint16_t)(raw.y >> 16));
+}
+template <typename T>
+DEVINL void gn4_store(T* p, const float* v);
+template <>
+DEVINL void gn4_store<float>(float* p, const float* v) {
+  *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+}
+template <>
+DEVINL void gn4_store<bf16_t>(bf16_t* p, const float* v) {
+  uint2 raw;
+  raw.x = (uint32_t)f32_to_bf16_bits(v[0]) | ((uint32_t)f32_to_bf16_bits(v[1]) << 16);
+  raw.y = (uint32_t)f32_to_bf16_bits(v[2]) | ((uint32_t)f32_to_bf16_bits(v[3]) << 16);
+  *reinterpret_cast<uint2*>(p) = raw;
+}
+
+// silu(z) or sigmoid(z)
+DEVINL float gn_act(float z, bool sigmoid) {
+  const float s = 1.0f / (1.0f + expf(-z));
+  return sigmoid ? s : z * s;
+}
+
+// out[t, h*dv + j] = o[t,h,j] / rms(o[t,h,:]) * w[j] * act(gate[t, h*dv + j]), w
+// null = no weight. lpr lanes per (token, head): VEC: 4 values per lane (dv a
+// multiple of 4, at most 256, rows aligned), lpr a power of two with 4 lpr >= dv;
+// else a wave per row.
+template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void gated_rmsnorm_kernel(
     T* __restrict__ out, const float* __restrict__ o, const T* __restrict__ gate,
-    int64_t gate_stride, const T* __restrict__ w, float eps, int rows, int H,
-    int dv) {
-  const int64_t row = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (row >= rows) return;
-  const int lane = threadIdx.x & 63;
-  const int64_t t = row / H;
-  const int h = row % H;
-  const float* x = o + row * dv;
-  float sq = 0.f;
-  for (int i = lane; i < dv; i += 64) sq += x[i] * x[i];
-  sq = wave_reduce_sum(sq);
-  const float rinv = 1.0f / sqrtf(sq / (float)dv + eps);
+    int64_t gate_stride, const T* __restrict__ w, float eps, int64_t rows, int H,
+    int dv, int lpr, int sigmoid) {
+  const int lane = threadIdx.x & 63, sub = lane % lpr;
+  const int64_t row =
+      ((int64_t)blockIdx.x * 4 + (threadIdx.x >> 6)) * (64 / lpr) + lane / lpr;
+  const bool on = row < rows;   // all lanes stay for the reductions
+  const int64_t r_ = on ? row : rows - 1;
+  const int64_t t = r_ / H;
+  const int h = (int)(r_ % H);
+  const float* x = o + r_ * dv;
   const T* gr = gate + t * gate_stride + h * dv;
-  T* dst = out + row * dv;
-  for (int i = lane; i < dv; i += 64) {
-    const float gv = ldf(gr + i);
-    const float sg = gv / (1.0f + expf(-gv));
-    stf(dst + i, x[i] * rinv * ldf(w + i) * sg);
+  T* dst = out + r_ * dv;
+  float v[4] = {0.f, 0.f, 0.f, 0.f};
+  float sq = 0.f;
+  if (VEC) {
+    if (sub * 4 < dv) gn4_load<float>(x + sub * 4, v);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) sq = fmaf(v[j], v[j], sq);
+  } else {
+    for (int i = sub; i < dv; i += 64) sq = fmaf(x[i], x[i], sq);
+  }
+  for (int off = lpr >> 1; off > 0; off >>= 1) sq += __shfl_xor(sq, off, 64);
+  if (!on) return;
+  const float r = 1.0f / sqrtf(sq / (float)dv + eps);
+  if (VEC) {
+    const int i = sub * 4;
+    if (i < dv) {
+      float gv[4], wv[4] = {1.f, 1.f, 1.f, 1.f};
+      gn4_load<T>(gr + i, gv);
+      if (w) gn4_load<T>(w + i, wv);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] = v[j] * r * wv[j] * gn_act(gv[j], sigmoid);
+      gn4_store<T>(dst + i, v);
+    }
+  } else {
+    for (int i = sub; i < dv; i += 64)
+      stf(dst + i, x[i] * r * (w ? ldf(w + i) : 1.f) * gn_act(ldf(gr + i), sigmoid));
+  }
+}
+
+// the same with ONE norm over a token's whole row of n = H dv values and a weight
+// that wide; a workgroup per token, the row in registers up to n = 4096 (VEC)
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void gated_rmsnorm_row_kernel(
+    T* __restrict__ out, const float* __restrict__ o, const T* __restrict__ gate,
+    int64_t gate_stride, const T* __restrict__ w, float eps, int n, int sigmoid) {
+  __shared__ float scratch[8];
+  const int64_t t = blockIdx.x;
+  const float* x = o + t * (int64_t)n;
+  const T* gr = gate + t * gate_stride;
+  T* dst = out + t * (int64_t)n;
+  float sq = 0.f;
+  if (VEC) {
+    float v[4][4];
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      const int i = (c * 256 + threadIdx.x) * 4;
+      if (i < n) {
+        gn4_load<float>(x + i, v[c]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) sq = fmaf(v[c][j], v[c][j], sq);
+      }
+    }
+    sq = block256_sum(sq, scratch);
+    const float r = 1.0f / sqrtf(sq / (float)n + eps);
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      const int i = (c * 256 + threadIdx.x) * 4;
+      if (i < n) {
+        float gv[4], wv[4] = {1.f, 1.f, 1.f, 1.f};
+        gn4_load<T>(gr + i, gv);
+        if (w) gn4_load<T>(w + i, wv);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[c][j] = v[c][j] * r * wv[j] * gn_act(gv[j], sigmoid);
+        gn4_store<T>(dst + i, v[c]);
+      }
+    }
+  } else {
+    for (int i = threadIdx.x; i < n; i += 256) sq = fmaf(x[i], x[i], sq);
+    sq = block256_sum(sq, scratch);
+    const float r = 1.0f / sqrtf(sq / (float)n + eps);
+    for (int i = threadIdx.x; i < n; i += 256)
+      stf(dst + i, x[i] * r * (w ? ldf(w + i) : 1.f) * gn_act(ldf(gr + i), sigmoid));
   }
 }
 
@@ -175,18 +277,48 @@ extern "C" void launch_gla_recurrence(
                         inv_tau, q_scale, stream);
 }
 
+template <typename T>
+static void launch_gated_rmsnorm_t(T* out, const float* o, const T* gate,
+                                   int64_t gate_stride, const T* w, float eps, int T_,
+                                   int H, int dv, int whole, int sigmoid,
+                                   hipStream_t stream) {
+  const int n = whole ? H * dv : dv;
+  const bool vec = n % 4 == 0 && n <= (whole ? 4096 : 256) && gate_stride % 4 == 0 &&
+                   ((uintptr_t)gate % (4 * sizeof(T))) == 0 &&
+                   ((uintptr_t)w % (4 * sizeof(T))) == 0;
+  if (whole) {
+    if (vec)
+      hipLaunchKernelGGL((gated_rmsnorm_row_kernel<T, true>), dim3(T_), dim3(256), 0,
+                         stream, out, o, gate, gate_stride, w, eps, n, sigmoid);
+    else
+      hipLaunchKernelGGL((gated_rmsnorm_row_kernel<T, false>), dim3(T_), dim3(256), 0,
+                         stream, out, o, gate, gate_stride, w, eps, n, sigmoid);
+    return;
+  }
+  int lpr = 64;
+  if (vec)
+    while (lpr > 1 && lpr * 2 >= dv) lpr >>= 1;   // the smallest with 4 lpr >= dv
+  const int64_t rows = (int64_t)T_ * H, per_block = 4 * (64 / lpr);
+  const dim3 grid((rows + per_block - 1) / per_block);
+  if (vec)
+    hipLaunchKernelGGL((gated_rmsnorm_kernel<T, true>), grid, dim3(256), 0, stream, out,
+                       o, gate, gate_stride, w, eps, rows, H, dv, lpr, sigmoid);
+  else
+    hipLaunchKernelGGL((gated_rmsnorm_kernel<T, false>), grid, dim3(256), 0, stream, out,
+                       o, gate, gate_stride, w, eps, rows, H, dv, lpr, sigmoid);
+}
+
 extern "C" void launch_gated_rmsnorm(void* out, const float* o, const void* gate,
                                      int64_t gate_stride, const void* w,
-                                     float eps, int rows, int H, int dv,
-                                     int kind, hipStream_t stream) {
-  if (rows == 0) return;
-  const dim3 grid((rows + 3) / 4);
+                                     float eps, int T_, int H, int dv, int whole,
+                                     int sigmoid, int kind, hipStream_t stream) {
+  if (T_ == 0 || H == 0) return;
   if (kind == 0)
-    hipLaunchKernelGGL((gated_rmsnorm_kernel<bf16_t>), grid, dim3(256), 0,
-                       stream, (bf16_t*)out, o, (const bf16_t*)gate, gate_stride,
-                       (const bf16_t*)w, eps, rows, H, dv);
+    launch_gated_rmsnorm_t<bf16_t>((bf16_t*)out, o, (const bf16_t*)gate, gate_stride,
+                                   (const bf16_t*)w, eps, T_, H, dv, whole, sigmoid,
+                                   stream);
   else
-    hipLaunchKernelGGL((gated_rmsnorm_kernel<float>), grid, dim3(256), 0, stream,
-                       (float*)out, o, (const float*)gate, gate_stride,
-                       (const float*)w, eps, rows, H, dv);
+    launch_gated_rmsnorm_t<float>((float*)out, o, (const float*)gate, gate_stride,
+                                  (const float*)w, eps, T_, H, dv, whole, sigmoid,
+                                  stream);
 }

@@ -2,6 +2,7 @@
 // the feed-forward run side by side on the same normed input), with an RMS
 // norm taken in groups; embedding with a hashed (previous token, token) pair
 // table; squared relu; rotation of attention results back by their position.
+// Also the residual step of layers that give both sublayers a norm of their own.
 //
 //   group_rmsnorm_add   : x <- x + (y1 + y2) in fp32, then the row is split
 //                         into `groups` equal consecutive parts, each divided
@@ -12,6 +13,11 @@
 //                         (16-byte accesses), each thread leaves the sum of
 //                         its 4 squares in LDS and one wave per group adds the
 //                         group's partial sums in a fixed order.
+//   parallel_rmsnorm_add: m = a, or scale * (a / rms(a) wa + b / rms(b) wb) for
+//                         two mixers side by side; x <- x + (m + f) in fp32; then
+//                         h_i = x / rms(x) * (offset + w_i) for the next layer's
+//                         mixer and feed-forward. One 256-thread workgroup per
+//                         token, every operand read once up to width 4096.
 //   pair_hash_embedding : out = table[id] * scale + pair[r] in fp32, r = (prev
 //                         * mul_prev + id * mul_cur) mod buckets, or the pair
 //                         table's last row for a token without a predecessor.
@@ -165,6 +171,184 @@ extern "C" void launch_group_rmsnorm_add(float* x, const void* y1,
     else GN_CALL(float, false);
   }
 #undef GN_CALL
+}
+
+// ---- parallel sublayers on norms of their own -----------------------------------
+
+// sums of two values over a 256-thread block; every thread gets both
+DEVINL void gn_sum2(float& a, float& b, float* scratch) {
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  a = wave_reduce_sum(a);
+  b = wave_reduce_sum(b);
+  if (lane == 0) {
+    scratch[2 * wid] = a;
+    scratch[2 * wid + 1] = b;
+  }
+  __syncthreads();
+  a = scratch[0] + scratch[2] + scratch[4] + scratch[6];
+  b = scratch[1] + scratch[3] + scratch[5] + scratch[7];
+}
+
+// VEC: W % 4 == 0, W <= 4096, rows 16-byte aligned (8-byte for bf16)
+template <typename T, typename F, bool VEC>
+__global__ __launch_bounds__(256) void parallel_rmsnorm_add_kernel(
+    float* __restrict__ x, const T* __restrict__ a, int64_t a_stride,
+    const T* __restrict__ b, int64_t b_stride, const T* __restrict__ wa,
+    const T* __restrict__ wb, float scale, const F* __restrict__ f, int64_t f_stride,
+    const T* __restrict__ w1, const T* __restrict__ w2, float eps, float offset,
+    T* __restrict__ h1, T* __restrict__ h2, int W) {
+  __shared__ float s_ab[8], s_x[8];
+  const int64_t row = blockIdx.x;
+  float* xr = x + row * (int64_t)W;
+  const T* ra = a ? a + row * a_stride : nullptr;
+  const T* rb = b ? b + row * b_stride : nullptr;
+  const F* rf = f ? f + row * f_stride : nullptr;
+  T* o1 = w1 ? h1 + row * (int64_t)W : nullptr;
+  T* o2 = w2 ? h2 + row * (int64_t)W : nullptr;
+  const float rw = 1.0f / (float)W;
+  if (VEC) {
+    float v[GN_MAXV][4], va[GN_MAXV][4], vb[GN_MAXV][4];
+    float sa = 0.f, sb = 0.f;
+#pragma unroll
+    for (int c = 0; c < GN_MAXV; ++c) {
+      const int i = (c * 256 + threadIdx.x) * 4;
+      if (i < W) {
+        gn_load4<float>(xr + i, v[c]);
+        if (ra) gn_load4<T>(ra + i, va[c]);
+        if (rb) {
+          gn_load4<T>(rb + i, vb[c]);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            sa = fmaf(va[c][j], va[c][j], sa);
+            sb = fmaf(vb[c][j], vb[c][j], sb);
+          }
+        }
+      }
+    }
+    if (rb) {
+      gn_sum2(sa, sb, s_ab);
+      sa = scale / sqrtf(sa * rw + eps);
+      sb = scale / sqrtf(sb * rw + eps);
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < GN_MAXV; ++c) {
+      const int i = (c * 256 + threadIdx.x) * 4;
+      if (i < W) {
+        float m[4] = {0.f, 0.f, 0.f, 0.f};
+        if (rb) {
+          float p[4], q[4];
+          gn_load4<T>(wa + i, p);
+          gn_load4<T>(wb + i, q);
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            m[j] = fmaf(va[c][j] * sa, p[j], vb[c][j] * sb * q[j]);
+        } else if (ra) {
+#pragma unroll
+          for (int j = 0; j < 4; ++j) m[j] = va[c][j];
+        }
+        if (rf) {
+          float q[4];
+          gn_load4<F>(rf + i, q);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) m[j] += q[j];
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          v[c][j] += m[j];
+          ss = fmaf(v[c][j], v[c][j], ss);
+        }
+        if (ra || rf) gn_store4<float>(xr + i, v[c]);
+      }
+    }
+    if (!o1 && !o2) return;
+    float none = 0.f;
+    gn_sum2(ss, none, s_x);
+    const float r = 1.0f / sqrtf(ss * rw + eps);
+#pragma unroll
+    for (int c = 0; c < GN_MAXV; ++c) {
+      const int i = (c * 256 + threadIdx.x) * 4;
+      if (i < W) {
+        float p[4], h[4];
+        if (o1) {
+          gn_load4<T>(w1 + i, p);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) h[j] = v[c][j] * r * (offset + p[j]);
+          gn_store4<T>(o1 + i, h);
+        }
+        if (o2) {
+          gn_load4<T>(w2 + i, p);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) h[j] = v[c][j] * r * (offset + p[j]);
+          gn_store4<T>(o2 + i, h);
+        }
+      }
+    }
+  } else {
+    float sa = 0.f, sb = 0.f;
+    if (rb) {
+      for (int i = threadIdx.x; i < W; i += 256) {
+        const float p = ldf(ra + i), q = ldf(rb + i);
+        sa = fmaf(p, p, sa);
+        sb = fmaf(q, q, sb);
+      }
+      gn_sum2(sa, sb, s_ab);
+      sa = scale / sqrtf(sa * rw + eps);
+      sb = scale / sqrtf(sb * rw + eps);
+    }
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < W; i += 256) {
+      float m = 0.f;
+      if (rb) m = fmaf(ldf(ra + i) * sa, ldf(wa + i), ldf(rb + i) * sb * ldf(wb + i));
+      else if (ra) m = ldf(ra + i);
+      if (rf) m += ldf(rf + i);
+      const float y = xr[i] + m;
+      ss = fmaf(y, y, ss);
+      if (ra || rf) xr[i] = y;
+    }
+    if (!o1 && !o2) return;
+    float none = 0.f;
+    gn_sum2(ss, none, s_x);
+    const float r = 1.0f / sqrtf(ss * rw + eps);
+    // every thread reads back what it stored itself
+    for (int i = threadIdx.x; i < W; i += 256) {
+      const float y = xr[i] * r;
+      if (o1) stf(o1 + i, y * (offset + ldf(w1 + i)));
+      if (o2) stf(o2 + i, y * (offset + ldf(w2 + i)));
+    }
+  }
+}
+
+// kind: activation type (0 bf16, 1 float); f_kind: type of f
+extern "C" void launch_parallel_rmsnorm_add(
+    float* x, const void* a, int64_t a_stride, const void* b, int64_t b_stride,
+    const void* wa, const void* wb, float scale, const void* f, int64_t f_stride,
+    int f_kind, const void* w1, const void* w2, float eps, float offset, void* h1,
+    void* h2, int rows, int W, int kind, hipStream_t stream) {
+  if (rows == 0) return;
+  const int esz = kind == 0 ? 2 : 4, fsz = f_kind == 0 ? 2 : 4;
+  auto ok = [](const void* p, int64_t stride, int sz) {
+    return p == nullptr || (stride % 4 == 0 && ((uintptr_t)p % (4 * sz)) == 0);
+  };
+  const bool vec = W % 4 == 0 && W <= 1024 * GN_MAXV && ok(a, a_stride, esz) &&
+                   ok(b, b_stride, esz) && ok(f, f_stride, fsz);
+#define PR_CALL(TT, FF, V)                                                        \
+  hipLaunchKernelGGL((parallel_rmsnorm_add_kernel<TT, FF, V>), dim3(rows),        \
+                     dim3(256), 0, stream, x, (const TT*)a, a_stride, (const TT*)b, \
+                     b_stride, (const TT*)wa, (const TT*)wb, scale, (const FF*)f, \
+                     f_stride, (const TT*)w1, (const TT*)w2, eps, offset, (TT*)h1, \
+                     (TT*)h2, W)
+  if (kind == 0 && f_kind == 0) {
+    if (vec) PR_CALL(bf16_t, bf16_t, true);
+    else PR_CALL(bf16_t, bf16_t, false);
+  } else if (kind == 0) {
+    if (vec) PR_CALL(bf16_t, float, true);
+    else PR_CALL(bf16_t, float, false);
+  } else {
+    if (vec) PR_CALL(float, float, true);
+    else PR_CALL(float, float, false);
+  }
+#undef PR_CALL
 }
 
 // ---- embedding with a hashed pair table -----------------------------------------

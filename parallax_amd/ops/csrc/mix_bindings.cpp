@@ -2,7 +2,8 @@
 // fp32-residual layer norm, sliding-window latent attention, gated linear
 // attention, sandwich RMS norm with depth averaging, row-cache attention
 // (differential / pooled sliding window), xIELU, hyper-connected streams,
-// matrix LSTM, softmax router. Every entry point checks shapes and types on the host before a
+// matrix LSTM, softmax router, parallel residual with two norms, short convolution,
+// fixed-decay linear attention, gated delta rule. Every entry point checks shapes and types on the host before a
 // launch; activation tensors are bf16 or float32 (one template instance each).
 
 #include <ATen/hip/HIPContext.h>
@@ -40,8 +41,24 @@ void launch_biased_glu(void*, const void*, int64_t, const void*, int, int, int,
 void launch_softcap_logits(float*, const void*, float, float, int64_t, int,
                            hipStream_t);
 void launch_small_linear(float*, const void*, int64_t, const void*, int, int,
-                         int, int64_t*, float*, const float*, int, int,
+                         int, int64_t*, float*, const float*, int, int, int, int,
                          hipStream_t);
+void launch_parallel_rmsnorm_add(float*, const void*, int64_t, const void*, int64_t,
+                                 const void*, const void*, float, const void*,
+                                 int64_t, int, const void*, const void*, float,
+                                 float, void*, void*, int, int, int, hipStream_t);
+void launch_short_conv(void*, const void*, int64_t, const void*, void*,
+                       const int64_t*, const int*, const int*, int, int, int, int,
+                       int, hipStream_t);
+void launch_rope_table(float*, const int*, const float*, int, int, hipStream_t);
+int linear_recurrence_chunk();
+void launch_linear_recurrence(float*, const void*, const void*, const void*,
+                              const int64_t*, float, float, int, const float*, int,
+                              const float*, int, const float*, const float*,
+                              const float*, float*, const int64_t*, const int*,
+                              const int*, int, int, int, int, int, float*, float*,
+                              float*, float*, float*, float*, int, int, int,
+                              hipStream_t);
 void launch_latent_gather(void*, void*, const void*, const int*, int, const int*,
                           int, int, int, int, int, hipStream_t);
 int latent_expanded_supported(int, int, int);
@@ -62,7 +79,8 @@ void launch_gla_recurrence(float*, const void*, const void*, const void*,
                            const int*, int, int, int, int, float, float, int,
                            hipStream_t);
 void launch_gated_rmsnorm(void*, const float*, const void*, int64_t,
-                          const void*, float, int, int, int, int, hipStream_t);
+                          const void*, float, int, int, int, int, int, int,
+                          hipStream_t);
 void launch_sandwich_rmsnorm(float*, const void*, int64_t, int, const void*,
                              float*, int64_t, int, const float*, const void*,
                              float, float, void*, const void*, const int*, int,
@@ -86,14 +104,15 @@ void launch_row_attention_prefill(void*, float*, const float*, const void*,
                                   int, const int*, int, int, int, int, int, int,
                                   int, int, int, int, float, float, float,
                                   float, float, const float*, const void*,
-                                  int64_t, int, const float*, int, int,
+                                  int64_t, int, int, const float*, int,
+                                  const float*, int, const float*, int, int,
                                   hipStream_t);
 void launch_row_attention(void*, float*, float*, const float*, const void*,
                           const float*, const int*, int, const int*, const int*,
                           int, int, int, int, int, int, int, int, int, int,
                           float, float, float, float, float, int, const float*,
-                          const void*, int64_t, int, const float*, int, int,
-                          hipStream_t);
+                          const void*, int64_t, int, int, const float*, int,
+                          const float*, int, const float*, int, hipStream_t);
 void launch_group_rmsnorm_add(float*, const void*, int64_t, const void*,
                               int64_t, const void*, float, void*, int, int,
                               int, int, hipStream_t);
@@ -349,9 +368,10 @@ void gla_recurrence(torch::Tensor o, torch::Tensor q, torch::Tensor k,
       dk, dv, (float)inv_tau, (float)q_scale, kind, cur_stream());
 }
 
-// o [T, H, dv] fp32, gate [T, H*dv], weight [dv] -> out [T, H*dv]
+// o [T, H, dv] fp32, gate [T, H*dv], weight [dv] ([H*dv] when whole) or empty ->
+// out [T, H*dv]
 void gated_rmsnorm(torch::Tensor out, torch::Tensor o, torch::Tensor gate,
-                   torch::Tensor weight, double eps) {
+                   torch::Tensor weight, double eps, bool whole, bool sigmoid) {
   const int kind = kind_of(gate, "gate");
   CHECK_F32C(o);
   TORCH_CHECK(o.dim() == 3);
@@ -360,11 +380,14 @@ void gated_rmsnorm(torch::Tensor out, torch::Tensor o, torch::Tensor gate,
               gate.stride(1) == 1);
   TORCH_CHECK(out.is_cuda() && out.scalar_type() == gate.scalar_type() &&
               out.is_contiguous() && out.numel() == (int64_t)T * H * dv);
-  TORCH_CHECK(weight.is_cuda() && weight.scalar_type() == gate.scalar_type() &&
-              weight.numel() == dv && weight.is_contiguous());
+  const bool has_w = weight.numel() > 0;
+  if (has_w)
+    TORCH_CHECK(weight.is_cuda() && weight.scalar_type() == gate.scalar_type() &&
+                weight.numel() == (whole ? (int64_t)H * dv : (int64_t)dv) &&
+                weight.is_contiguous());
   launch_gated_rmsnorm(out.data_ptr(), o.data_ptr<float>(), gate.data_ptr(),
-                       gate.stride(0), weight.data_ptr(), (float)eps, T * H, H,
-                       dv, kind, cur_stream());
+                       gate.stride(0), has_w ? weight.data_ptr() : nullptr, (float)eps,
+                       T, H, dv, whole ? 1 : 0, sigmoid ? 1 : 0, kind, cur_stream());
 }
 
 // x [T, W] fp32 (in place); y [T, W] (row stride free) + w_branch [W] or
@@ -570,11 +593,13 @@ void row_attention(torch::Tensor out, torch::Tensor q, torch::Tensor cache,
                    double norm_eps, double out_mult, int64_t max_keys,
                    torch::Tensor query_bounds, torch::Tensor head_bias,
                    torch::Tensor gate, int64_t value_col, torch::Tensor rot_cs,
-                   bool rot_interleaved) {
+                   bool rot_interleaved, torch::Tensor dist_bias,
+                   torch::Tensor sink, bool bf16_q) {
   const int kind = kind_of(cache, "cache");
   CHECK_F32C(q);
   // head_bias [H] fp32: sigmoid(score + head_bias[h]) weights, not normalised;
-  // gate [T, H] (cache type, row stride free): result times sigmoid(gate)
+  // gate [T, H] or [T, H * dv] (cache type, row stride free): result times
+  // sigmoid(gate), per head or per element
   const bool has_bias = head_bias.numel() > 0, has_gate = gate.numel() > 0;
   if (has_bias) {
     CHECK_F32C(head_bias);
@@ -583,7 +608,24 @@ void row_attention(torch::Tensor out, torch::Tensor q, torch::Tensor cache,
   if (has_gate)
     TORCH_CHECK(gate.is_cuda() && gate.scalar_type() == cache.scalar_type() &&
                 gate.dim() == 2 && gate.size(0) == q.size(0) &&
-                gate.size(1) == H && gate.stride(1) == 1, "gate");
+                (gate.size(1) == H || gate.size(1) == H * dv) &&
+                gate.stride(1) == 1, "gate");
+  const int gate_w = has_gate ? (int)(gate.size(1) / H) : 0;
+  // dist_bias [H, n] fp32, sink [H] fp32: softmax weights, one map, no pooled rows
+  const bool has_rel = dist_bias.numel() > 0, has_sink = sink.numel() > 0;
+  if (has_rel || has_sink)
+    TORCH_CHECK(M == 1 && !has_bias && !(window > 0 && P > 0), "distance bias, sinks");
+  if (has_rel) {
+    CHECK_F32C(dist_bias);
+    TORCH_CHECK(dist_bias.dim() == 2 && dist_bias.size(0) == H, "distance bias");
+  }
+  if (has_sink) {
+    CHECK_F32C(sink);
+    TORCH_CHECK(sink.numel() == H, "sinks");
+  }
+  const float* rel_p = has_rel ? dist_bias.data_ptr<float>() : nullptr;
+  const int n_rel = has_rel ? (int)dist_bias.size(1) : 1;
+  const float* sink_p = has_sink ? sink.data_ptr<float>() : nullptr;
   const float* bias_p = has_bias ? head_bias.data_ptr<float>() : nullptr;
   const void* gate_p = has_gate ? gate.data_ptr() : nullptr;
   const int64_t gate_stride = has_gate ? gate.stride(0) : 0;
@@ -666,8 +708,9 @@ void row_attention(torch::Tensor out, torch::Tensor q, torch::Tensor cache,
         (T + 31) / 32 + B, (int)H, (int)G, (int)M, (int)d, (int)dv,
         (int)cache.size(1), per_page, (int)window, has_pool ? (int)P : 0,
         (float)scale, (float)softcap, (float)lam, (float)norm_eps,
-        (float)out_mult, bias_p, gate_p, gate_stride, vbase,
-        turn_after ? nullptr : rot_p, rot_inter, kind, cur_stream());
+        (float)out_mult, bias_p, gate_p, gate_stride, gate_w, vbase,
+        turn_after ? nullptr : rot_p, rot_inter, rel_p, n_rel, sink_p,
+        bf16_q ? 1 : 0, kind, cur_stream());
     if (turn_after)
       launch_rotate_heads_table(out.data_ptr(), tmp.data_ptr<float>(), rot_p,
                                 (int)H, (int)dv, rot_inter, -1.0f, T,
@@ -702,8 +745,8 @@ void row_attention(torch::Tensor out, torch::Tensor q, torch::Tensor cache,
       positions.data_ptr<int>(), T, (int)H, (int)G, (int)M, (int)d, (int)dv,
       (int)cache.size(1), per_page, (int)window, has_pool ? (int)P : 0,
       (float)scale, (float)softcap, (float)lam, (float)norm_eps,
-      (float)out_mult, splits, bias_p, gate_p, gate_stride, vbase, rot_p,
-      rot_inter, kind, cur_stream());
+      (float)out_mult, splits, bias_p, gate_p, gate_stride, gate_w, vbase, rot_p,
+      rot_inter, rel_p, n_rel, sink_p, kind, cur_stream());
 }
 
 // x [T, W] fp32 (updated in place when y1 is given); y1, y2 [T, W] of the
@@ -1002,17 +1045,19 @@ void linear_f32(torch::Tensor out, torch::Tensor x, torch::Tensor w) {
   TORCH_CHECK(out.dim() == 2 && out.size(0) == T && out.size(1) == N);
   launch_small_linear(out.data_ptr<float>(), x.data_ptr(), x.stride(0),
                       w.data_ptr(), T, N, (int)x.size(1), nullptr, nullptr,
-                      nullptr, 0, 0, cur_stream());
+                      nullptr, 0, 0, 1, 1, cur_stream());
 }
 
 // ids [T, top] int64, wts [T, top] fp32, rest [T, N - E] fp32
 void route_softmax(torch::Tensor ids, torch::Tensor wts, torch::Tensor rest,
                    torch::Tensor x, torch::Tensor w, torch::Tensor bias,
-                   int64_t E, int64_t top) {
+                   int64_t E, int64_t top, int64_t groups, int64_t keep) {
   check_small_linear(x, w);
   const int T = x.size(0), N = w.size(0);
   TORCH_CHECK(E >= 1 && E <= N && N <= 240, "router rows");
   TORCH_CHECK(top >= 1 && top <= E && top <= 64, "experts per token");
+  TORCH_CHECK(groups >= 1 && groups <= 64 && E % groups == 0 && keep >= 1 &&
+              keep <= groups && top <= E / groups * keep, "expert groups");
   CHECK_I64(ids);
   CHECK_F32C(wts);
   CHECK_F32C(rest);
@@ -1027,7 +1072,8 @@ void route_softmax(torch::Tensor ids, torch::Tensor wts, torch::Tensor rest,
                       w.data_ptr(), T, N, (int)x.size(1),
                       ids.data_ptr<int64_t>(), wts.data_ptr<float>(),
                       has_b ? bias.data_ptr<float>() : nullptr, (int)E,
-                      (int)top, cur_stream());
+                      (int)top, keep < groups ? (int)groups : 1, (int)keep,
+                      cur_stream());
 }
 
 // q, k [T, H * d], v, g [T, H * dv] (row strides free), gates [T, 2 H] fp32,
@@ -1163,7 +1209,218 @@ void latent_expanded_attention(torch::Tensor out, torch::Tensor q,
       cur_stream());
 }
 
+// x [T, W] fp32 in place; a, b [T, W] (activation type, row strides free) or empty;
+// wa, wb [W] with b; f [T, W] (activation type or fp32) or empty; w1, h1 and w2, h2
+// [W], [T, W] or empty each
+void parallel_rmsnorm_add(torch::Tensor x, torch::Tensor a, torch::Tensor b,
+                          torch::Tensor wa, torch::Tensor wb, double scale,
+                          torch::Tensor f, torch::Tensor w1, torch::Tensor w2,
+                          double eps, double offset, torch::Tensor h1,
+                          torch::Tensor h2) {
+  CHECK_F32C(x);
+  TORCH_CHECK(x.dim() == 2);
+  const int T = x.size(0), W = x.size(1);
+  if (T == 0) return;
+  const int kind = kind_of(h1, "h1");   // the activation type, also when empty
+  auto rows = [&](const torch::Tensor& t, const char* what) {
+    TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.size(0) == T && t.size(1) == W &&
+                t.stride(1) == 1, what);
+  };
+  auto vec = [&](const torch::Tensor& t, const char* what) {
+    TORCH_CHECK(kind_of(t, what) == kind && t.is_contiguous() && t.numel() == W, what);
+  };
+  const bool has_a = a.numel() > 0, has_b = b.numel() > 0, has_f = f.numel() > 0;
+  const bool has1 = w1.numel() > 0, has2 = w2.numel() > 0;
+  TORCH_CHECK(has_a || !has_b, "b without a");
+  if (has_a) {
+    rows(a, "a");
+    TORCH_CHECK(kind_of(a, "a") == kind, "a");
+  }
+  if (has_b) {
+    rows(b, "b");
+    TORCH_CHECK(kind_of(b, "b") == kind, "b");
+    vec(wa, "wa");
+    vec(wb, "wb");
+  }
+  int f_kind = kind;
+  if (has_f) {
+    rows(f, "f");
+    f_kind = kind_of(f, "f");
+    TORCH_CHECK(kind == 0 || f_kind == 1, "fp32 stacks take fp32 branches");
+  }
+  for (const auto& p : {std::make_pair(&w1, &h1), std::make_pair(&w2, &h2)}) {
+    if (p.first->numel() == 0) continue;
+    vec(*p.first, "norm weight");
+    rows(*p.second, "h");
+    TORCH_CHECK(p.second->is_contiguous() && kind_of(*p.second, "h") == kind, "h");
+  }
+  launch_parallel_rmsnorm_add(
+      x.data_ptr<float>(), has_a ? a.data_ptr() : nullptr, has_a ? a.stride(0) : 0,
+      has_b ? b.data_ptr() : nullptr, has_b ? b.stride(0) : 0,
+      has_b ? wa.data_ptr() : nullptr, has_b ? wb.data_ptr() : nullptr, (float)scale,
+      has_f ? f.data_ptr() : nullptr, has_f ? f.stride(0) : 0, f_kind,
+      has1 ? w1.data_ptr() : nullptr, has2 ? w2.data_ptr() : nullptr, (float)eps,
+      (float)offset, has1 ? h1.data_ptr() : nullptr, has2 ? h2.data_ptr() : nullptr, T,
+      W, kind, cur_stream());
+}
+
+// x [T, C] (row stride free), weight [C, taps], state [slots, C, taps - 1] (all of
+// one type), slots [B] int64, cu [B + 1] int32 or empty (one token per sequence)
+void short_conv(torch::Tensor out, torch::Tensor x, torch::Tensor weight,
+                torch::Tensor state, torch::Tensor slots, torch::Tensor cu,
+                torch::Tensor positions) {
+  const int kind = kind_of(x, "x");
+  TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1 && weight.dim() == 2);
+  const int T = x.size(0), C = x.size(1), taps = weight.size(1);
+  TORCH_CHECK(taps >= 1 && taps <= 64, "convolution taps");
+  TORCH_CHECK(kind_of(weight, "weight") == kind && weight.is_contiguous() &&
+              weight.size(0) == C, "convolution weight");
+  TORCH_CHECK(kind_of(state, "state") == kind && state.is_contiguous() &&
+              state.dim() == 3 && state.size(1) == C && state.size(2) == taps - 1,
+              "convolution state");
+  TORCH_CHECK(kind_of(out, "out") == kind && out.is_contiguous() && out.dim() == 2 &&
+              out.size(0) == T && out.size(1) == C);
+  CHECK_I64(slots);
+  CHECK_I32(positions);
+  TORCH_CHECK(positions.numel() == T);
+  const int B = slots.numel();
+  const bool has_cu = cu.numel() > 0;
+  if (has_cu) {
+    CHECK_I32(cu);
+    TORCH_CHECK(cu.numel() == B + 1);
+  } else {
+    TORCH_CHECK(B == T, "without cu every sequence brings one token");
+  }
+  launch_short_conv(out.data_ptr(), x.data_ptr(), x.stride(0), weight.data_ptr(),
+                    state.data_ptr(), slots.data_ptr<int64_t>(),
+                    has_cu ? cu.data_ptr<int>() : nullptr, positions.data_ptr<int>(), T,
+                    B, C, taps, kind, cur_stream());
+}
+
+// out [T, 2 n] fp32, freq [n] fp32
+void rope_table(torch::Tensor out, torch::Tensor positions, torch::Tensor freq) {
+  CHECK_F32C(out);
+  CHECK_F32C(freq);
+  CHECK_I32(positions);
+  const int T = positions.numel(), n = freq.numel();
+  TORCH_CHECK(out.dim() == 2 && out.size(0) == T && out.size(1) == 2 * n);
+  launch_rope_table(out.data_ptr<float>(), positions.data_ptr<int>(),
+                    freq.data_ptr<float>(), n, T, cur_stream());
+}
+
+// The two forms of linear_recurrence.hip. q, k [T, G, d], v [T, H, dv] (token and
+// head strides free), state [slots, H, d, dv] fp32, o [T, H, dv] fp32.
+static void linear_recurrence(torch::Tensor o, torch::Tensor q, torch::Tensor k,
+                              torch::Tensor v, double q_scale, double k_scale,
+                              bool silu, const float* cs, int n_rot, const float* pw,
+                              int pw_n, const float* gates, const float* a_log,
+                              const float* dt_bias, torch::Tensor state,
+                              torch::Tensor slots, torch::Tensor cu,
+                              torch::Tensor positions) {
+  const int kind = kind_of(q, "q");
+  CHECK_F32C(o);
+  CHECK_F32C(state);
+  TORCH_CHECK(q.dim() == 3 && v.dim() == 3 && state.dim() == 4);
+  const int T = q.size(0), G = q.size(1), d = q.size(2);
+  const int H = v.size(1), dv = v.size(2);
+  TORCH_CHECK(G >= 1 && d >= 1 && dv >= 1 && H % G == 0, "heads");
+  TORCH_CHECK(k.is_cuda() && k.scalar_type() == q.scalar_type() &&
+              k.sizes() == q.sizes() && v.is_cuda() &&
+              v.scalar_type() == q.scalar_type() && v.size(0) == T);
+  TORCH_CHECK(q.stride(2) == 1 && k.stride(2) == 1 && v.stride(2) == 1, "strides");
+  TORCH_CHECK(state.size(1) == H && state.size(2) == d && state.size(3) == dv &&
+              o.dim() == 3 && o.size(0) == T && o.size(1) == H && o.size(2) == dv,
+              "state and result");
+  TORCH_CHECK(d <= 1024, "key width above 1024 is not supported");
+  CHECK_I64(slots);
+  CHECK_I32(positions);
+  TORCH_CHECK(positions.numel() == T);
+  const int B = slots.numel();
+  const bool has_cu = cu.numel() > 0;
+  if (has_cu) {
+    CHECK_I32(cu);
+    TORCH_CHECK(cu.numel() == B + 1);
+  } else {
+    TORCH_CHECK(B == T, "without cu every sequence brings one token");
+  }
+  if (T == 0) return;
+  const int L = linear_recurrence_chunk();
+  const int64_t strides[6] = {q.stride(0), q.stride(1), k.stride(0),
+                              k.stride(1), v.stride(0), v.stride(1)};
+  // portions of some length run in chunks; few tokens a sequence, one by one
+  int tiles = 0, vec = 0;
+  torch::Tensor qp, kp, P, M, e;
+  if (has_cu && d <= 256 && T >= 16 * B) {
+    TORCH_CHECK(pw == nullptr || pw_n > L, "powers of the decays");
+    tiles = (T + L - 1) / L + B;
+    vec = d % 8 == 0 && dv % 8 == 0;
+    for (int64_t s : strides) vec = vec && s % 8 == 0;
+    for (const torch::Tensor* t : {&q, &k, &v})
+      vec = vec && ((uintptr_t)t->data_ptr() % 16) == 0;
+    qp = torch::empty({(int64_t)T, G, d}, state.options());
+    kp = torch::empty({(int64_t)T, G, d}, state.options());
+    P = torch::empty({(int64_t)tiles, H, L, L}, state.options());
+    if (gates) M = torch::empty({(int64_t)tiles, H, L, L}, state.options());
+    e = torch::empty({2, (int64_t)tiles, H, L}, state.options());
+  }
+  float* ep = tiles ? e.data_ptr<float>() : nullptr;
+  launch_linear_recurrence(
+      o.data_ptr<float>(), q.data_ptr(), k.data_ptr(), v.data_ptr(), strides,
+      (float)q_scale, (float)k_scale, silu ? 1 : 0, cs, n_rot, pw, pw_n, gates, a_log,
+      dt_bias, state.data_ptr<float>(), slots.data_ptr<int64_t>(),
+      has_cu ? cu.data_ptr<int>() : nullptr, positions.data_ptr<int>(), B, H, G, d, dv,
+      tiles ? qp.data_ptr<float>() : nullptr, tiles ? kp.data_ptr<float>() : nullptr,
+      tiles ? P.data_ptr<float>() : nullptr,
+      tiles && gates ? M.data_ptr<float>() : nullptr, ep,
+      tiles ? ep + (int64_t)tiles * H * L : nullptr, tiles, vec, kind, cur_stream());
+}
+
+// powers [H, N] fp32: 0th, 1st, ... power of every head's decay; rot_cs [T, n_rot]
+// fp32 (cos, sin pairs) or empty
+void decay_attention(torch::Tensor o, torch::Tensor q, torch::Tensor k, torch::Tensor v,
+                     torch::Tensor powers, double k_scale, bool silu,
+                     torch::Tensor rot_cs, torch::Tensor state, torch::Tensor slots,
+                     torch::Tensor cu, torch::Tensor positions) {
+  CHECK_F32C(powers);
+  TORCH_CHECK(q.dim() == 3 && v.dim() == 3 && v.size(1) == q.size(1) &&
+              powers.dim() == 2 && powers.size(0) == q.size(1) && powers.size(1) >= 2,
+              "decays");
+  const bool has_rot = rot_cs.numel() > 0;
+  if (has_rot) {
+    CHECK_F32C(rot_cs);
+    TORCH_CHECK(rot_cs.dim() == 2 && rot_cs.size(0) == q.size(0) &&
+                rot_cs.size(1) % 2 == 0 && rot_cs.size(1) <= q.size(2), "rotation");
+  }
+  linear_recurrence(o, q, k, v, 1.0, k_scale, silu,
+                    has_rot ? rot_cs.data_ptr<float>() : nullptr,
+                    has_rot ? (int)rot_cs.size(1) : 0, powers.data_ptr<float>(),
+                    (int)powers.size(1), nullptr, nullptr, nullptr, state, slots, cu,
+                    positions);
+}
+
+// gates [T, 2 H] fp32 (step size | decay pre-activations), a_log, dt_bias [H] fp32
+void gated_delta_rule(torch::Tensor o, torch::Tensor q, torch::Tensor k,
+                      torch::Tensor v, torch::Tensor gates, torch::Tensor a_log,
+                      torch::Tensor dt_bias, torch::Tensor state, torch::Tensor slots,
+                      torch::Tensor cu, torch::Tensor positions) {
+  CHECK_F32C(gates);
+  CHECK_F32C(a_log);
+  CHECK_F32C(dt_bias);
+  TORCH_CHECK(q.dim() == 3 && v.dim() == 3);
+  const int64_t H = v.size(1);
+  TORCH_CHECK(gates.dim() == 2 && gates.size(0) == q.size(0) && gates.size(1) == 2 * H &&
+              a_log.numel() == H && dt_bias.numel() == H, "gates");
+  linear_recurrence(o, q, k, v, 1.0 / std::sqrt((double)q.size(2)), 1.0, false, nullptr,
+                    0, nullptr, 0, gates.data_ptr<float>(), a_log.data_ptr<float>(),
+                    dt_bias.data_ptr<float>(), state, slots, cu, positions);
+}
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  m.def("parallel_rmsnorm_add", &parallel_rmsnorm_add);
+  m.def("short_conv", &short_conv);
+  m.def("rope_table", &rope_table);
+  m.def("decay_attention", &decay_attention);
+  m.def("gated_delta_rule", &gated_delta_rule);
   m.def("add_layernorm", &add_layernorm);
   m.def("latent_kv_store", &latent_kv_store);
   m.def("rope_rows", &rope_rows);

@@ -1,6 +1,6 @@
 // Grouped-head attention over a row-per-token paged cache: softmax weights,
 // or sigmoid(score + per-head bias) weights that are not normalised over the
-// keys; optionally a per-head sigmoid gate on the result.
+// keys; optionally a sigmoid gate on the result, per head or per element.
 //
 // A cache row holds, for one token, the keys of all kv heads and then the
 // values of all kv heads: [G x M x d | G x dv], M = score maps per head (1, or
@@ -40,6 +40,10 @@
 //                       head_bias[h]); the running maximum is pinned at 0
 //                       and the denominator at 1, so partial results of
 //                       waves and key shares simply add up.
+//   distance bias     : dist_bias[h, min(pos - j, n - 1)] added to the scaled
+//                       score of key j. sink: a key-less term exp(sink[h]) of
+//                       the denominator, where wave 0 of share 0 starts its
+//                       running maximum. Both with softmax weights only.
 #include "seq_common.h"
 
 #define RA_WAVES 4
@@ -407,15 +411,19 @@ DEVINL void ra_dot(const TK* __restrict__ key, const float* __restrict__ qs,
   }
 }
 
+DEVINL float ra_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
+
 // The shared end of the main kernel and the reduce kernel: one wave turns the
 // unnormalised sums of one head (M maps, acc[m * acc_stride + f], softmax
-// denominators l[m]) into the head's output row.
+// denominators l[m]) into the head's output row. gate_row: the head's dv gate
+// pre-activations (element-wise gate) or null.
 template <typename T, int M>
 DEVINL void ra_epilogue(T* __restrict__ dst, float* __restrict__ dst32,
                         const float* __restrict__ acc,
                         int acc_stride, const float* l, int dv, float lam,
                         float norm_eps, float out_mult, float post,
-                        const float* __restrict__ rcs, int rot_inter) {
+                        const float* __restrict__ rcs, int rot_inter,
+                        const T* __restrict__ gate_row) {
   const int lane = threadIdx.x & 63;
   const float i0 = 1.0f / l[0];
   const float i1 = M == 2 ? lam / l[1] : 0.f;
@@ -453,19 +461,26 @@ DEVINL void ra_epilogue(T* __restrict__ dst, float* __restrict__ dst32,
   for (int c = 0; c < 4; ++c) {
     const int f = lane + 64 * c;
     if (f < dv) {
-      if (dst32) dst32[f] = o[c] * r;
-      else stf(dst + f, o[c] * r);
+      float v = o[c] * r;
+      if (gate_row) v *= ra_sigmoid(ldf(gate_row + f));
+      if (dst32) dst32[f] = v;
+      else stf(dst + f, v);
     }
   }
 }
 
-DEVINL float ra_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
-
-// sigmoid(gate[t, h]) or 1
+// sigmoid(gate[t, h]) or 1 (gate_w: gate pre-activations per head, 1 or dv)
 template <typename T>
-DEVINL float ra_gate(const T* __restrict__ gate, int64_t gate_stride, int64_t t,
-                     int h) {
-  return gate ? ra_sigmoid(ldf(gate + t * gate_stride + h)) : 1.0f;
+DEVINL float ra_gate(const T* __restrict__ gate, int64_t gate_stride, int gate_w,
+                     int64_t t, int h) {
+  return gate && gate_w == 1 ? ra_sigmoid(ldf(gate + t * gate_stride + h)) : 1.0f;
+}
+
+// the head's row of an element-wise gate, or null
+template <typename T>
+DEVINL const T* ra_gate_row(const T* gate, int64_t gate_stride, int gate_w, int64_t t,
+                            int h) {
+  return gate && gate_w > 1 ? gate + t * gate_stride + (int64_t)h * gate_w : nullptr;
 }
 
 // part layout: [T, H, splits, M, 2 + dv]: running max, denominator, sums
@@ -481,8 +496,10 @@ __global__ __launch_bounds__(256) void row_attention_kernel(
     int G, int d, int dv, int block_size, int per_page, int window, int P,
     float scale, float softcap, float lam, float norm_eps, float out_mult,
     int splits, int FL, const float* __restrict__ head_bias,
-    const T* __restrict__ gate, int64_t gate_stride, int vbase,
-    const float* __restrict__ rot_cs, int rot_inter) {
+    const T* __restrict__ gate, int64_t gate_stride, int gate_w, int vbase,
+    const float* __restrict__ rot_cs, int rot_inter,
+    const float* __restrict__ dist_bias, int n_bias,
+    const float* __restrict__ sink) {
   constexpr int NQ = HB * M;
   extern __shared__ float lds[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -524,6 +541,10 @@ __global__ __launch_bounds__(256) void row_attention_kernel(
     hb[n] = sig ? head_bias[g * rep + min(r0 + n / M, rep - 1)] : 0.f;
     mx[n] = sig ? 0.f : -INFINITY;
     l[n] = 0.f;
+    if (sink != nullptr && split == 0 && wave == 0) {
+      mx[n] = sink[g * rep + min(r0 + n / M, rep - 1)];
+      l[n] = 1.f;
+    }
 #pragma unroll
     for (int i = 0; i < 4; ++i) acc[n][i] = 0.f;
   }
@@ -578,6 +599,9 @@ __global__ __launch_bounds__(256) void row_attention_kernel(
     for (int n = 0; n < NQ; ++n) {
       float sc = s[n] * scale;
       if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
+      if (dist_bias != nullptr && valid)   // no pooled rows: key u is lo + u
+        sc += dist_bias[(int64_t)(g * rep + min(r0 + n / M, rep - 1)) * n_bias +
+                        min(pos - lo - u, n_bias - 1)];
       float p;
       if (sig) {
         p = valid ? ra_sigmoid(sc + hb[n]) : 0.f;
@@ -698,8 +722,9 @@ __global__ __launch_bounds__(256) void row_attention_kernel(
                         out32 ? out32 + (t * H + h) * (int64_t)dv : nullptr,
                         oacc + hh * M * dvp, dvp,
                         lg, dv, lam, norm_eps, out_mult,
-                        ra_gate<T>(gate, gate_stride, t, h),
-                        rot_cs ? rot_cs + t * dv : nullptr, rot_inter);
+                        ra_gate<T>(gate, gate_stride, gate_w, t, h),
+                        rot_cs ? rot_cs + t * dv : nullptr, rot_inter,
+                        ra_gate_row<T>(gate, gate_stride, gate_w, t, h));
     } else {
 #pragma unroll
       for (int m = 0; m < M; ++m) {
@@ -722,7 +747,7 @@ __global__ __launch_bounds__(64) void row_attention_reduce_kernel(
     T* __restrict__ out, float* __restrict__ out32,
     const float* __restrict__ part, int dv, int splits,
     float lam, float norm_eps, float out_mult, int H, int sig,
-    const T* __restrict__ gate, int64_t gate_stride,
+    const T* __restrict__ gate, int64_t gate_stride, int gate_w,
     const float* __restrict__ rot_cs, int rot_inter) {
   extern __shared__ float lds[];  // [M][dvp] sums | [M][64] weights
   const int64_t th = blockIdx.x;
@@ -770,8 +795,10 @@ __global__ __launch_bounds__(64) void row_attention_reduce_kernel(
   ra_epilogue<T, M>(out + th * (int64_t)dv,
                     out32 ? out32 + th * (int64_t)dv : nullptr, lds, dvp, lg,
                     dv, lam, norm_eps,
-                    out_mult, ra_gate<T>(gate, gate_stride, th / H, (int)(th % H)),
-                    rot_cs ? rot_cs + (th / H) * dv : nullptr, rot_inter);
+                    out_mult,
+                    ra_gate<T>(gate, gate_stride, gate_w, th / H, (int)(th % H)),
+                    rot_cs ? rot_cs + (th / H) * dv : nullptr, rot_inter,
+                    ra_gate_row<T>(gate, gate_stride, gate_w, th / H, (int)(th % H)));
 }
 
 struct RaArgs {
@@ -791,9 +818,13 @@ struct RaArgs {
   const float* head_bias;
   const void* gate;
   int64_t gate_stride;
+  int gate_w;
   int vbase;
   const float* rot_cs;
   int rot_inter;
+  const float* dist_bias;
+  int n_bias;
+  const float* sink;
   hipStream_t stream;
 };
 
@@ -819,8 +850,8 @@ static void launch_ra_hb(const RaArgs& a) {
                      a.positions, a.H, a.G, a.d, a.dv, a.block_size,          \
                      a.per_page, a.window, a.P, a.scale, a.softcap, a.lam,    \
                      a.norm_eps, a.out_mult, a.splits, FL, a.head_bias,       \
-                     (const T*)a.gate, a.gate_stride, a.vbase, a.rot_cs,      \
-                     a.rot_inter)
+                     (const T*)a.gate, a.gate_stride, a.gate_w, a.vbase,      \
+                     a.rot_cs, a.rot_inter, a.dist_bias, a.n_bias, a.sink)
   const bool pooled = a.pool != nullptr && a.window > 0 && a.P > 0;
   if (vec) {
     if (pooled) RA_CALL(true, true);
@@ -836,7 +867,8 @@ static void launch_ra_hb(const RaArgs& a) {
                        a.stream, (T*)a.out, a.out32, a.part, a.dv, a.splits,
                        a.lam,
                        a.norm_eps, a.out_mult, a.H, a.head_bias != nullptr,
-                       (const T*)a.gate, a.gate_stride, a.rot_cs, a.rot_inter);
+                       (const T*)a.gate, a.gate_stride, a.gate_w, a.rot_cs,
+                       a.rot_inter);
 }
 
 template <typename T, int M>
@@ -858,13 +890,15 @@ extern "C" void launch_row_attention(
     const int* positions, int T_, int H, int G, int M, int d, int dv,
     int block_size, int per_page, int window, int P, float scale, float softcap,
     float lam, float norm_eps, float out_mult, int splits,
-    const float* head_bias, const void* gate, int64_t gate_stride, int vbase,
-    const float* rot_cs, int rot_inter, int kind, hipStream_t stream) {
+    const float* head_bias, const void* gate, int64_t gate_stride, int gate_w,
+    int vbase, const float* rot_cs, int rot_inter, const float* dist_bias,
+    int n_bias, const float* sink, int kind, hipStream_t stream) {
   if (T_ == 0) return;
   const RaArgs a{out, out32, part, q, cache, pool, block_tables, bt_stride, token_seq,
                  positions, T_, H, G, d, dv, block_size, per_page, window, P,
                  scale, softcap, lam, norm_eps, out_mult, splits, head_bias,
-                 gate, gate_stride, vbase, rot_cs, rot_inter, stream};
+                 gate, gate_stride, gate_w, vbase, rot_cs, rot_inter, dist_bias,
+                 n_bias, sink, stream};
   if (kind == 0) {
     if (M == 1) launch_ra_m<bf16_t, 1>(a);
     else launch_ra_m<bf16_t, 2>(a);

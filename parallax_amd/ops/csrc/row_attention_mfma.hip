@@ -28,9 +28,14 @@
 // norm over the value width; division by the softmax sum; optional sigmoid
 // gate per (token, head)) works on columns, i.e. per lane pair, too.
 //
-// SIG instantiations replace the softmax by sigmoid(score + head_bias[h])
-// weights that are not normalised over the keys: no running maximum, no
-// rescaling of the accumulators, masked keys weigh 0.
+// Key weights (template parameter W): RM_SOFTMAX; RM_SIGMOID replaces the softmax
+// by sigmoid(score + head_bias[h]) weights that are not normalised over the keys:
+// no running maximum, no rescaling of the accumulators, masked keys weigh 0;
+// RM_BIAS is the softmax with dist_bias[h, min(distance, n - 1)] added to the
+// scaled score (steps whose keys are all farther than the table is long add one
+// constant) and a key-less term exp(sink[h]) in the denominator, where the running
+// maximum starts. RM_BIAS_BF16Q is RM_BIAS for queries that are bf16 numbers
+// themselves (bf16 kernel only: one part of three is enough).
 #include <cstdlib>
 #include <type_traits>
 
@@ -41,6 +46,11 @@ typedef float f32x16v __attribute__((ext_vector_type(16)));
 #define RM_Q 32     // queries per workgroup
 #define RM_K 32     // keys per step
 #define RM_PAD 4    // LDS row padding (floats)
+
+#define RM_SOFTMAX 0
+#define RM_SIGMOID 1
+#define RM_BIAS 2
+#define RM_BIAS_BF16Q 3
 
 template <typename T>
 DEVINL void rm_load8(const T* p, float* v);
@@ -96,11 +106,11 @@ DEVINL float rm_tanh(float x) {
 
 // sigmoid through the same two hardware approximations
 DEVINL float rm_sigmoid(float x) { return __frcp_rn(1.0f + __expf(-x)); }
-// once per (token, head): the library exponential
+// outside the inner loops: the library exponential
 DEVINL float rm_sigmoid_exact(float x) { return 1.0f / (1.0f + expf(-x)); }
 
 // D: padded key width (64 | 128), DVB: 32-wide blocks of the padded value width
-template <typename T, int M, int D, int DVB, bool SIG>
+template <typename T, int M, int D, int DVB, int W>
 __global__ __launch_bounds__(256, 2) void row_attention_prefill_kernel(
     T* __restrict__ out, float* __restrict__ out32, const float* __restrict__ q, const T* __restrict__ cache,
     const float* __restrict__ pool, const int* __restrict__ block_tables,
@@ -109,8 +119,10 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_kernel(
     int block_size, int per_page, int window, int P, float scale, float softcap,
     float lam, float norm_eps, float out_mult,
     const float* __restrict__ head_bias, const T* __restrict__ gate,
-    int64_t gate_stride, int vbase, const float* __restrict__ rot_cs,
-    int rot_inter) {
+    int64_t gate_stride, int gate_w, int vbase, const float* __restrict__ rot_cs,
+    int rot_inter, const float* __restrict__ dist_bias, int n_bias,
+    const float* __restrict__ sink) {
+  constexpr bool SIG = W == RM_SIGMOID, REL = W >= RM_BIAS;
   constexpr int DV = DVB * 32;
   constexpr int KS = D + RM_PAD, VS = DV + RM_PAD;
   constexpr int HW = 4 / M;  // heads per workgroup
@@ -175,6 +187,12 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_kernel(
   float mx = -INFINITY, l = 0.f;
   const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
   const float hbias = SIG ? head_bias[h] : 0.f;
+  const float* brow = (REL && dist_bias) ? dist_bias + (int64_t)h * n_bias : nullptr;
+  const float bfar = brow ? brow[n_bias - 1] : 0.f;
+  if (REL && sink) {
+    mx = sink[h];
+    l = 1.f;
+  }
 
   // staging role: 8 threads per key row, 8 features each at a time
   const int srow = threadIdx.x >> 3, ssub = threadIdx.x & 7;
@@ -333,7 +351,22 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_kernel(
           }
       }
     } else {
-    if (interior) {
+    if (REL) {
+      // one score map, no pooled rows: key u of the step is at jt0 + (u - u0)
+      const bool far = p0 - (jt0 + RM_K - 1) >= n_bias - 1;
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const int u = 8 * (i >> 2) + 4 * half + (i & 3), jt = jt0 + u;
+        const bool vis = interior || (jt <= pq && (window == 0 || pq - jt < window) &&
+                                      qvalid && u0 + u < nk);
+        float sc = S[i] * scale;
+        if (softcap > 0.f) sc = softcap * rm_tanh(sc * inv_cap);
+        if (brow) sc += far ? bfar : brow[min(max(pq - jt, 0), n_bias - 1)];
+        sc = vis ? sc : -INFINITY;
+        S[i] = sc;
+        tmax = fmaxf(tmax, sc);
+      }
+    } else if (interior) {
 #pragma unroll
       for (int i = 0; i < 16; ++i) {
         float sc = S[i] * scale;
@@ -472,8 +505,18 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_kernel(
     r = out_mult / sqrtf(ss / (float)dv + norm_eps);
   }
   if (!stream_on || !qvalid) return;
-  if (gate != nullptr)
+  if (gate != nullptr && gate_w == 1)
     r *= rm_sigmoid_exact(ldf(gate + (int64_t)(t0 + col) * gate_stride + h));
+  if (gate != nullptr && gate_w > 1) {   // a gate per element of the head
+    const T* gr = gate + (int64_t)(t0 + col) * gate_stride + (int64_t)h * gate_w;
+#pragma unroll
+    for (int k = 0; k < DVB; ++k)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const int f = 32 * k + 8 * (i >> 2) + 4 * half + (i & 3);
+        if (f < dv) acc[k][i] *= rm_sigmoid(ldf(gr + f));
+      }
+  }
   const int64_t o0 = ((int64_t)(t0 + col) * H + h) * dv;
   if (out32 != nullptr) {
 #pragma unroll
@@ -531,7 +574,7 @@ DEVINL void rb_split3(float x, short& hi, short& mid, short& lo) {
 #define RB_KPAD 8   // bf16 elements of padding per K row (16 bytes)
 #define RB_VS 36    // bf16 elements per transposed V row: 32 keys + 4 (72 bytes)
 
-template <int D, int DVB, bool SIG>
+template <int D, int DVB, int W>
 __global__ __launch_bounds__(256, 2) void row_attention_prefill_bf16_kernel(
     bf16_t* __restrict__ out, float* __restrict__ out32, const float* __restrict__ q,
     const bf16_t* __restrict__ cache, const int* __restrict__ block_tables,
@@ -539,8 +582,12 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_bf16_kernel(
     const int* __restrict__ positions, int H, int G, int d, int dv,
     int block_size, int window, float scale, float softcap, float norm_eps,
     float out_mult, const float* __restrict__ head_bias,
-    const bf16_t* __restrict__ gate, int64_t gate_stride, int vbase,
-    const float* __restrict__ rot_cs, int rot_inter) {
+    const bf16_t* __restrict__ gate, int64_t gate_stride, int gate_w, int vbase,
+    const float* __restrict__ rot_cs, int rot_inter,
+    const float* __restrict__ dist_bias, int n_bias,
+    const float* __restrict__ sink) {
+  constexpr bool SIG = W == RM_SIGMOID, REL = W >= RM_BIAS;
+  constexpr bool Q3 = W != RM_BIAS_BF16Q;   // queries need all three parts
   constexpr int DV = DVB * 32;
   constexpr int KS = D + RB_KPAD;
   constexpr int HW = 4;  // heads per workgroup
@@ -604,6 +651,12 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_bf16_kernel(
   float mx = -INFINITY, l = 0.f;
   const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
   const float hbias = SIG ? head_bias[h] : 0.f;
+  const float* brow = (REL && dist_bias) ? dist_bias + (int64_t)h * n_bias : nullptr;
+  const float bfar = brow ? brow[n_bias - 1] : 0.f;
+  if (REL && sink) {
+    mx = sink[h];
+    l = 1.f;
+  }
 
   // staging role: 8 threads per key row, 8 elements each at a time
   const int srow = threadIdx.x >> 3, ssub = threadIdx.x & 7;
@@ -667,8 +720,10 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_bf16_kernel(
       for (int s = 0; s < D / 16; ++s) {
         const bf16x8v a = *reinterpret_cast<const bf16x8v*>(krow + 16 * s);
         S = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, qh[s], S, 0, 0, 0);
-        S = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, qm[s], S, 0, 0, 0);
-        S = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, ql[s], S, 0, 0, 0);
+        if (Q3) {
+          S = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, qm[s], S, 0, 0, 0);
+          S = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, ql[s], S, 0, 0, 0);
+        }
       }
     }
     // ---- mask, soft cap, weights (column = query, 16 keys in-lane) ---------------
@@ -691,6 +746,7 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_bf16_kernel(
         }
     } else {
       float tmax = -INFINITY;
+      const bool far = REL && p0 - (jt0 + RM_K - 1) >= n_bias - 1;
 #pragma unroll
       for (int i = 0; i < 4; ++i)
 #pragma unroll
@@ -701,6 +757,7 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_bf16_kernel(
                                         qvalid && u < nk);
           float sc = S[4 * i + j] * scale;
           if (softcap > 0.f) sc = softcap * rm_tanh(sc * inv_cap);
+          if (REL && brow) sc += far ? bfar : brow[min(max(pq - jt, 0), n_bias - 1)];
           sc = vis ? sc : -INFINITY;
           S[4 * i + j] = sc;
           tmax = fmaxf(tmax, sc);
@@ -800,8 +857,18 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_bf16_kernel(
     r = out_mult / sqrtf(ss / (float)dv + norm_eps);
   }
   if (!stream_on || !qvalid) return;
-  if (gate != nullptr)
+  if (gate != nullptr && gate_w == 1)
     r *= rm_sigmoid_exact(ldf(gate + (int64_t)(t0 + col) * gate_stride + h));
+  if (gate != nullptr && gate_w > 1) {   // a gate per element of the head
+    const bf16_t* gr = gate + (int64_t)(t0 + col) * gate_stride + (int64_t)h * gate_w;
+#pragma unroll
+    for (int k = 0; k < DVB; ++k)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const int f = 32 * k + 8 * (i >> 2) + 4 * half + (i & 3);
+        if (f < dv) acc[k][i] *= rm_sigmoid(ldf(gr + f));
+      }
+  }
   const int64_t o0 = ((int64_t)(t0 + col) * H + h) * dv;
 #pragma unroll
   for (int k = 0; k < DVB; ++k)
@@ -831,9 +898,14 @@ struct RmArgs {
   const float* head_bias;
   const void* gate;
   int64_t gate_stride;
+  int gate_w;
   int vbase;
   const float* rot_cs;
   int rot_inter;
+  const float* dist_bias;
+  int n_bias;
+  const float* sink;
+  int bf16_q;   // the queries are bf16 numbers
   hipStream_t stream;
 };
 
@@ -846,29 +918,30 @@ static bool rm_split_bf16() {
   return on;
 }
 
-template <int D, int DVB, bool SIG>
+template <int D, int DVB, int W>
 static void launch_rb(const RmArgs& a) {
   constexpr int DV = DVB * 32;
   const int rep = a.H / a.G;
   const size_t shm = sizeof(bf16_t) * ((size_t)RM_K * (D + RB_KPAD) + (size_t)DV * RB_VS);
   const dim3 grid(a.tiles, a.G * ((rep + 3) / 4));
-  hipLaunchKernelGGL((row_attention_prefill_bf16_kernel<D, DVB, SIG>), grid,
+  hipLaunchKernelGGL((row_attention_prefill_bf16_kernel<D, DVB, W>), grid,
                      dim3(256), shm, a.stream, (bf16_t*)a.out, a.out32, a.q,
                      (const bf16_t*)a.cache, a.block_tables, a.bt_stride, a.cu,
                      a.B, a.positions, a.H, a.G, a.d, a.dv, a.block_size,
                      a.window, a.scale, a.softcap, a.norm_eps, a.out_mult,
-                     a.head_bias, (const bf16_t*)a.gate, a.gate_stride, a.vbase,
-                     a.rot_cs, a.rot_inter);
+                     a.head_bias, (const bf16_t*)a.gate, a.gate_stride, a.gate_w,
+                     a.vbase, a.rot_cs, a.rot_inter, a.dist_bias, a.n_bias, a.sink);
 }
 
-template <typename T, int M, int D, int DVB, bool SIG>
+template <typename T, int M, int D, int DVB, int W>
 static void launch_rm_k(const RmArgs& a) {
   constexpr int DV = DVB * 32;
   // bf16 rows, one score map, no pooled rows, value tiles up to 128: the
   // exact three-part products on the bf16 matrix cores
   if constexpr (std::is_same<T, bf16_t>::value && M == 1 && DVB <= 4) {
     if (a.P == 0 && rm_split_bf16()) {
-      launch_rb<D, DVB, SIG>(a);
+      if (W == RM_BIAS && a.bf16_q) launch_rb<D, DVB, W == RM_BIAS ? RM_BIAS_BF16Q : W>(a);
+      else launch_rb<D, DVB, W>(a);
       return;
     }
   }
@@ -883,25 +956,28 @@ static void launch_rm_k(const RmArgs& a) {
     static bool raised = false;
     if (!raised) {
       (void)hipFuncSetAttribute(
-          reinterpret_cast<const void*>(&row_attention_prefill_kernel<T, M, D, DVB, SIG>),
+          reinterpret_cast<const void*>(&row_attention_prefill_kernel<T, M, D, DVB, W>),
           hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024);
       raised = true;
     }
   }
-  hipLaunchKernelGGL((row_attention_prefill_kernel<T, M, D, DVB, SIG>), grid,
+  hipLaunchKernelGGL((row_attention_prefill_kernel<T, M, D, DVB, W>), grid,
                      dim3(256), shm, a.stream, (T*)a.out, a.out32, a.q,
                      (const T*)a.cache, a.pool, a.block_tables, a.bt_stride,
                      a.cu, a.B, a.positions, a.H, a.G, a.d, a.dv, a.block_size,
                      a.per_page, a.window, a.P, a.scale, a.softcap, a.lam,
                      a.norm_eps, a.out_mult, a.head_bias, (const T*)a.gate,
-                     a.gate_stride, a.vbase, a.rot_cs, a.rot_inter);
+                     a.gate_stride, a.gate_w, a.vbase, a.rot_cs, a.rot_inter,
+                     a.dist_bias, a.n_bias, a.sink);
 }
 
-// sigmoid weights come with one score map only
+// sigmoid weights, distance bias and sinks come with one score map only
 template <typename T, int M, int D, int DVB>
 static void launch_rm(const RmArgs& a) {
-  if (M == 1 && a.head_bias != nullptr) launch_rm_k<T, 1, D, DVB, true>(a);
-  else launch_rm_k<T, M, D, DVB, false>(a);
+  if (M == 1 && a.head_bias != nullptr) launch_rm_k<T, 1, D, DVB, RM_SIGMOID>(a);
+  else if (M == 1 && (a.dist_bias != nullptr || a.sink != nullptr))
+    launch_rm_k<T, 1, D, DVB, RM_BIAS>(a);
+  else launch_rm_k<T, M, D, DVB, RM_SOFTMAX>(a);
 }
 
 template <typename T, int M, int D>
@@ -937,13 +1013,15 @@ extern "C" void launch_row_attention_prefill(
     const int* positions, int tiles, int H, int G, int M, int d, int dv,
     int block_size, int per_page, int window, int P, float scale, float softcap,
     float lam, float norm_eps, float out_mult, const float* head_bias,
-    const void* gate, int64_t gate_stride, int vbase, const float* rot_cs,
-    int rot_inter, int kind, hipStream_t stream) {
+    const void* gate, int64_t gate_stride, int gate_w, int vbase,
+    const float* rot_cs, int rot_inter, const float* dist_bias, int n_bias,
+    const float* sink, int bf16_q, int kind, hipStream_t stream) {
   if (tiles == 0) return;
   const RmArgs a{out, out32, q, cache, pool, block_tables, bt_stride, cu, B, positions,
                  tiles, H, G, d, dv, block_size, per_page, window, P, scale,
                  softcap, lam, norm_eps, out_mult, head_bias, gate, gate_stride,
-                 vbase, rot_cs, rot_inter, stream};
+                 gate_w, vbase, rot_cs, rot_inter, dist_bias, n_bias, sink, bf16_q,
+                 stream};
   if (kind == 0) {
     if (M == 1) launch_rm_m<bf16_t, 1>(a);
     else launch_rm_m<bf16_t, 2>(a);

@@ -4,7 +4,9 @@
 //   linear_f32    : out [T, N] fp32 = x [T, K] bf16 . w [N, K]^T bf16.
 //   route_softmax : rows 0 .. E of w are experts: z = x w^T + bias, the `top`
 //                   largest (lower index first among equals), weights = softmax
-//                   over those; rows E .. N are handed out as fp32 outputs.
+//                   over those; rows E .. N are handed out as fp32 outputs. With
+//                   groups > 1 the experts form equal runs of neighbours and only
+//                   those of the `keep` runs with the largest single logit count.
 //
 // One workgroup takes 16 tokens and up to 16 NT columns. Its NW waves share out
 // the contraction (wave w takes every NW-th block of 32) on the bf16 matrix
@@ -37,7 +39,7 @@ __global__ __launch_bounds__(NW * 64) void small_linear_kernel(
     float* __restrict__ out, const bf16_t* __restrict__ x, int64_t x_stride,
     const bf16_t* __restrict__ w, int T_, int N, int K,
     int64_t* __restrict__ ids, float* __restrict__ wts,
-    const float* __restrict__ bias, int E, int top) {
+    const float* __restrict__ bias, int E, int top, int groups, int keep) {
   constexpr int NP = NT * 16 + 1;
   extern __shared__ float red[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -96,6 +98,25 @@ __global__ __launch_bounds__(NW * 64) void small_linear_kernel(
       const int e = lane + 64 * c;
       v[c] = e < E ? red[m * NP + e] : -INFINITY;
     }
+    if (groups > 1) {
+      // lane = group (at most 64): its largest logit, then its rank among the
+      // groups (lower index first among equals)
+      const int gs = E / groups;
+      float best = -INFINITY;
+      if (lane < groups)
+        for (int i = 0; i < gs; ++i) best = fmaxf(best, red[m * NP + lane * gs + i]);
+      int rank = 0;
+      for (int o = 0; o < groups; ++o) {
+        const float ob = __shfl(best, o, 64);
+        rank += ob > best || (ob == best && o < lane);
+      }
+      const unsigned long long in = __ballot(lane < groups && rank < keep);
+#pragma unroll
+      for (int c = 0; c < EC; ++c) {
+        const int e = lane + 64 * c;
+        if (e < E && !((in >> (e / gs)) & 1)) v[c] = -INFINITY;
+      }
+    }
     float mine = -INFINITY;  // lane r keeps the r-th choice's logit
     int mine_id = 0;
     for (int r = 0; r < top; ++r) {
@@ -137,15 +158,15 @@ __global__ __launch_bounds__(NW * 64) void small_linear_kernel(
 template <int NT>
 static void launch_sl(float* out, const bf16_t* x, int64_t x_stride,
                       const bf16_t* w, int T_, int N, int K, int64_t* ids,
-                      float* wts, const float* bias, int E, int top, bool vec,
-                      hipStream_t stream) {
+                      float* wts, const float* bias, int E, int top, int groups,
+                      int keep, bool vec, hipStream_t stream) {
   const dim3 grid((T_ + SL_TOK - 1) / SL_TOK, (N + NT * 16 - 1) / (NT * 16));
   constexpr int NW = NT <= 4 ? 8 : 4;   // partial sums within 64 KB of LDS
   const size_t shm = sizeof(float) * NW * SL_TOK * (NT * 16 + 1);
 #define SL_CALL(V, R)                                                         \
   hipLaunchKernelGGL((small_linear_kernel<NT, NW, V, R>), grid, dim3(NW * 64), \
                      shm, stream, out, x, x_stride, w, T_, N, K, ids, wts, bias, E, \
-                     top)
+                     top, groups, keep)
   if (ids != nullptr) {
     if (vec) SL_CALL(true, true);
     else SL_CALL(false, true);
@@ -160,13 +181,14 @@ static void launch_sl(float* out, const bf16_t* x, int64_t x_stride,
 extern "C" void launch_small_linear(float* out, const void* x, int64_t x_stride,
                                     const void* w, int T_, int N, int K,
                                     int64_t* ids, float* wts, const float* bias,
-                                    int E, int top, hipStream_t stream) {
+                                    int E, int top, int groups, int keep,
+                                    hipStream_t stream) {
   if (T_ == 0 || N == 0) return;
   const bf16_t* xp = (const bf16_t*)x;
   const bf16_t* wp = (const bf16_t*)w;
   const bool vec = K % 8 == 0 && x_stride % 8 == 0 && ((uintptr_t)x % 16) == 0 &&
                    ((uintptr_t)w % 16) == 0;
-#define SL_ARGS out, xp, x_stride, wp, T_, N, K, ids, wts, bias, E, top, vec, stream
+#define SL_ARGS out, xp, x_stride, wp, T_, N, K, ids, wts, bias, E, top, groups, keep, vec, stream
   if (N <= 16) launch_sl<1>(SL_ARGS);
   else if (N <= 32) launch_sl<2>(SL_ARGS);
   else if (N <= 64 || ids == nullptr) launch_sl<4>(SL_ARGS);

@@ -5,7 +5,9 @@ pooled sliding window / sigmoid-weighted with an output gate) and xIELU;
 post-norm residual step, minGRU scan and the clamped gated linear unit;
 grouped RMS norm over a parallel residual, hashed pair embedding, squared relu
 and the rotation of head rows by position; hyper-connected residual streams,
-matrix LSTM, softmax router, biased gated linear unit.
+matrix LSTM, softmax router, biased gated linear unit; parallel residual with
+two norms, short convolution, linear attention with a fixed decay, gated delta
+rule.
 
 GPU tensors go to the hand-written gfx950 kernels of the in-tree extension
 ``parallax_amd.ops._mix`` (bf16 or float32 activations; scores, norms, decays
@@ -192,14 +194,20 @@ def gla_recurrence(q, k, v, z, z_bias, state, slots, cu, positions, inv_tau,
     return o
 
 
-def gated_rmsnorm(o, gate, weight, eps, out_dtype):
-    """Per-head RMS norm of o [T, H, dv] (fp32) with a weight shared by heads,
-    times silu(gate) -> [T, H*dv] of out_dtype."""
+def gated_rmsnorm(o, gate, weight, eps, out_dtype, whole=False, act="silu"):
+    """RMS norm of o [T, H, dv] (fp32) per head with a weight [dv] shared by
+    heads, or, with whole, over all heads together with a weight [H * dv]
+    (weight None: none), times silu(gate) or sigmoid(gate) -> [T, H*dv] of
+    out_dtype."""
+    if act not in ("silu", "sigmoid"):
+        raise ValueError(f"unknown gate activation {act!r}")
     if not o.is_cuda:
-        return ref.gated_rmsnorm(o, gate, weight, eps, out_dtype)
+        return ref.gated_rmsnorm(o, gate, weight, eps, out_dtype, whole, act)
     T, H, dv = o.shape
     out = torch.empty(T, H * dv, dtype=out_dtype, device=o.device)
-    _mix_ext().gated_rmsnorm(out, o, gate, weight, float(eps))
+    _mix_ext().gated_rmsnorm(out, o, gate,
+                             weight if weight is not None else _empty(gate),
+                             float(eps), bool(whole), act == "sigmoid")
     return out
 
 
@@ -292,15 +300,20 @@ def row_attention(q, cache, pool, block_tables, token_seq, positions, heads,
                   softcap, lam, norm_eps, out_mult, out_dtype, max_seq_len=0,
                   query_bounds=None, head_bias=None, gate=None,
                   shared_kv=False, out_rot_cs=None, out_rot_interleaved=False,
-                  value_col=0):
+                  value_col=0, dist_bias=None, sink=None, bf16_queries=False):
     """Attention of fp32 queries over paged cache rows [keys | values] with
     grouped heads: full causal (window 0) or a sliding window with pooled
     blocks beyond it, optional tanh soft cap, one or two score maps per head
     (two combine as a1 - lam * a2), optional RMS norm of each head's result.
     Key weights: softmax, or, with head_bias [heads] fp32, sigmoid(score +
     head_bias[h]) without normalisation over the keys (one map only). gate
-    [T, heads] (fp32 pre-activations): head h's result is multiplied by
-    sigmoid(gate[t, h]). max_seq_len: the longest context of the batch as the host
+    [T, heads] (pre-activations): head h's result is multiplied by
+    sigmoid(gate[t, h]); gate [T, heads * vdim]: element by element. dist_bias
+    [heads, N] fp32: a key n positions back gets dist_bias[h, min(n, N - 1)]
+    added to its scaled score (softmax weights, one map, no pooled rows). sink
+    [heads] fp32: the softmax's denominator also holds exp(sink[h]) (same
+    conditions). bf16_queries: every query element is a bf16 number (saves work
+    where that matters; anything else in q would be cut off). max_seq_len: the longest context of the batch as the host
     knows it (0 = the block tables' capacity); it only sizes the split of
     long key ranges over workgroups. query_bounds [B+1] int32 (prompt portions:
     tokens of sequence b are query_bounds[b] .. query_bounds[b+1], at
@@ -318,9 +331,13 @@ def row_attention(q, cache, pool, block_tables, token_seq, positions, heads,
                                  window, pool_tokens, scale, softcap, lam,
                                  norm_eps, out_mult, out_dtype, head_bias, gate,
                                  shared_kv, out_rot_cs, out_rot_interleaved,
-                                 value_col)
+                                 value_col, dist_bias, sink)
     if head_bias is not None and maps != 1:
         raise ValueError("sigmoid key weights take one score map per head")
+    if (dist_bias is not None or sink is not None) and (
+            head_bias is not None or maps != 1 or pool is not None):
+        raise ValueError("distance bias and sinks come with softmax weights, one "
+                         "score map and no pooled rows")
     out = torch.empty(q.shape[0], heads * vdim, dtype=out_dtype, device=q.device)
     ef = torch.empty(0, dtype=torch.float32, device=q.device)
     _mix_ext().row_attention(
@@ -338,6 +355,8 @@ def row_attention(q, cache, pool, block_tables, token_seq, positions, heads,
         head_bias if head_bias is not None else ef,
         gate if gate is not None else ef, int(value_col) if shared_kv else -1,
         out_rot_cs if out_rot_cs is not None else ef, bool(out_rot_interleaved),
+        dist_bias if dist_bias is not None else ef,
+        sink if sink is not None else ef, bool(bf16_queries),
     )
     return out
 
@@ -549,28 +568,31 @@ def linear_f32(x, weight):
 
 ROUTE_MAX_ROWS = 240   # rows of the routing kernel's weight
 ROUTE_MAX_TOP = 64     # experts it chooses per token
+ROUTE_MAX_GROUPS = 64  # groups of experts it tells apart
 
 
-def route_softmax(x, weight, bias, experts, top):
+def route_softmax(x, weight, bias, experts, top, groups=1, keep=1):
     """Router: z = x W[:experts]^T + bias in fp32, the `top` largest, weights =
     softmax over those; rows of weight after the experts come back as plain
-    fp32 outputs. One kernel for bf16 activations and up to ROUTE_MAX_ROWS
+    fp32 outputs. groups > 1: only experts of the `keep` best of `groups` equal
+    runs of neighbours (by the largest logit of each) can be chosen. One kernel for bf16 activations and up to ROUTE_MAX_ROWS
     rows. Returns (ids [T, top] int64, weights [T, top] fp32, rest [T, N -
     experts] fp32). bias [experts] fp32 or None."""
     if not x.is_cuda:
-        return ref.route_softmax(x, weight, bias, experts, top)
+        return ref.route_softmax(x, weight, bias, experts, top, groups, keep)
     T, N = x.shape[0], weight.shape[0]
-    if x.dtype == torch.float32 or N > ROUTE_MAX_ROWS or top > ROUTE_MAX_TOP:
+    if x.dtype == torch.float32 or N > ROUTE_MAX_ROWS or top > ROUTE_MAX_TOP \
+            or groups > ROUTE_MAX_GROUPS:
         z = linear_f32(x, weight)
         zr = z[:, :experts] if bias is None else z[:, :experts] + bias
-        val, ids = zr.topk(top, dim=-1)
+        val, ids = ref.limit_to_groups(zr, groups, keep).topk(top, dim=-1)
         return ids, torch.softmax(val, dim=-1), z[:, experts:].contiguous()
     ids = torch.empty(T, top, dtype=torch.int64, device=x.device)
     wts = torch.empty(T, top, dtype=torch.float32, device=x.device)
     rest = torch.empty(T, N - experts, dtype=torch.float32, device=x.device)
     _mix_ext().route_softmax(ids, wts, rest, x, weight,
                              bias if bias is not None else _empty(wts),
-                             int(experts), int(top))
+                             int(experts), int(top), int(groups), int(keep))
     return ids, wts, rest
 
 
@@ -597,3 +619,104 @@ def softcap_logits(x, scale, cap):
     out = torch.empty(x.shape, dtype=torch.float32, device=x.device)
     _mix_ext().softcap_logits(out, x.contiguous(), float(scale), float(cap))
     return out
+
+
+# -- parallel layers with two norms, short convolution, decaying linear attention,
+# gated delta rule ------------------------------------------------------------------
+
+
+def parallel_rmsnorm_add(x, a, b, wa, wb, scale, f, w1, w2, eps, offset, out_dtype):
+    """One residual step around a mixer and a feed-forward that run side by
+    side on two norms of the same stream, one kernel; x [T, W] fp32 (in place):
+      m = a, or scale * (a / rms(a) * wa + b / rms(b) * wb) with two mixers
+      x <- x + (m + f),   h_i = x / rms(x) * (offset + w_i)
+    a, b in the activation dtype, f in it or fp32 (a None: no mixer result; f
+    None: no feed-forward). Returns (h1, h2) in out_dtype, None where w_i is."""
+    if not x.is_cuda:
+        return ref.parallel_rmsnorm_add(x, a, b, wa, wb, scale, f, w1, w2, eps,
+                                        offset, out_dtype)
+    e = _empty(x, out_dtype)
+    h1, h2 = (torch.empty(x.shape, dtype=out_dtype, device=x.device)
+              if w is not None else None for w in (w1, w2))
+
+    def opt(t):
+        return t if t is not None else e
+
+    _mix_ext().parallel_rmsnorm_add(
+        x, opt(a), opt(b), opt(wa) if b is not None else e,
+        opt(wb) if b is not None else e, float(scale), opt(f), opt(w1), opt(w2),
+        float(eps), float(offset), opt(h1), opt(h2))
+    return h1, h2
+
+
+def short_conv(x, weight, state, slots, cu, positions, out_dtype):
+    """Causal depthwise convolution of every channel with its own taps, then
+    silu, over packed sequences. x [T, C] (row stride free), weight [C, taps]
+    (last column: the current token's); state [slots, C, taps - 1] (the
+    activation dtype) holds the inputs before the portion (zeros when it begins
+    at position 0) and receives the portion's last ones. cu [B+1] int32 token
+    bounds (None: one token each). Returns [T, C]."""
+    if not x.is_cuda:
+        return ref.short_conv(x, weight, state, slots, cu, positions, out_dtype)
+    out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
+    _mix_ext().short_conv(out, x, weight, state, slots,
+                          cu if cu is not None else _empty(positions), positions)
+    return out
+
+
+def rope_table(positions, freq):
+    """fp32 [T, 2 n]: the tokens' (cos, sin) of pos * freq[i], angles in fp32."""
+    if not positions.is_cuda:
+        return ref.rope_table(positions, freq)
+    out = torch.empty(positions.shape[0], 2 * freq.shape[0], dtype=torch.float32,
+                      device=positions.device)
+    _mix_ext().rope_table(out, positions, freq)
+    return out
+
+
+# tokens the chunked kernels take at a time: powers of a decay go that far
+DECAY_CHUNK = 32
+
+
+def decay_powers(decay) -> torch.Tensor:
+    """fp32 [H, DECAY_CHUNK + 1]: powers 0, 1, ... of every decay (rounded once)."""
+    d = torch.tensor([float(x) for x in decay], dtype=torch.float64)
+    n = torch.arange(DECAY_CHUNK + 1, dtype=torch.float64)
+    return (d.unsqueeze(-1) ** n).float().contiguous()
+
+
+def decay_attention(q, k, v, powers, k_scale, silu, rot_cs, state, slots, cu,
+                    positions):
+    """Linear attention S_t = decay_h S_(t-1) + k_t v_t^T, o_t = S_t^T q_t over
+    packed sequences. q, k [T, H, d], v [T, H, dv] as projected (token and head
+    strides free); silu: all three pass silu; rot_cs [T, 2 n] (see rope_table):
+    q and k are rotated on their first 2 n dimensions (pairs i, i + n); k is
+    multiplied by k_scale. powers [H, DECAY_CHUNK + 1] fp32 (decay_powers) hold
+    the decays in column 1; the fp32 state [slots, H, d, dv] is read (or started from zero at position 0) and written back. cu [B+1] int32
+    token bounds (None: one token each). Everything fp32. Returns [T, H, dv]."""
+    if not q.is_cuda:
+        return ref.decay_attention(q, k, v, powers[:, 1], k_scale, silu, rot_cs,
+                                   state, slots, cu, positions)
+    o = torch.empty(v.shape, dtype=torch.float32, device=q.device)
+    _mix_ext().decay_attention(
+        o, q, k, v, powers, float(k_scale), bool(silu),
+        rot_cs if rot_cs is not None else _empty(q, torch.float32), state, slots,
+        cu if cu is not None else _empty(positions), positions)
+    return o
+
+
+def gated_delta_rule(q, k, v, gates, a_log, dt_bias, state, slots, cu, positions):
+    """Gated delta rule over packed sequences: q, k [T, G, d], v [T, H, dv]
+    (strides free; head h reads q/k head h // (H / G)), gates [T, 2 H] fp32 =
+    [step size | decay] pre-activations, a_log, dt_bias [H] fp32. Unit q and k
+    (q also times d^-1/2), beta = sigmoid, g = exp(-exp(a_log) softplus(. +
+    dt_bias)); S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q, all
+    fp32. State and cu as in decay_attention. Returns fp32 [T, H, dv]."""
+    if not q.is_cuda:
+        return ref.gated_delta_rule(q, k, v, gates, a_log, dt_bias, state, slots,
+                                    cu, positions)
+    o = torch.empty(v.shape, dtype=torch.float32, device=q.device)
+    _mix_ext().gated_delta_rule(
+        o, q, k, v, gates, a_log, dt_bias, state, slots,
+        cu if cu is not None else _empty(positions), positions)
+    return o

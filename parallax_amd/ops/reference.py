@@ -704,11 +704,18 @@ def gla_recurrence(q, k, v, z, z_bias, state, slots, cu, positions, inv_tau,
     return o
 
 
-def gated_rmsnorm(o, gate, weight, eps, out_dtype):
+def gated_rmsnorm(o, gate, weight, eps, out_dtype, whole=False, act="silu"):
+    """o [T, H, dv] fp32 divided by its RMS per head (whole: over all heads
+    together), times weight [dv] ([H * dv] when whole; None: no weight), times
+    act(gate) with act 'silu' or 'sigmoid'."""
     T, H, dv = o.shape
-    x = o / torch.sqrt((o * o).mean(-1, keepdim=True) + eps) * weight.float()
-    g = gate.float().view(T, H, dv)
-    return (x * torch.nn.functional.silu(g)).view(T, H * dv).to(out_dtype)
+    x = o.reshape(T, 1, H * dv) if whole else o
+    x = x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
+    if weight is not None:
+        x = x * weight.float()
+    g = gate.float().reshape(x.shape)
+    g = torch.nn.functional.silu(g) if act == "silu" else torch.sigmoid(g)
+    return (x * g).reshape(T, H * dv).to(out_dtype)
 
 
 # -- row-cache attention mixers: sandwich RMS norm with depth averaging,
@@ -852,7 +859,8 @@ def row_attention(q, cache, pool, block_tables, token_seq, positions, heads,
                   kv_heads, maps, dim, vdim, window, pool_tokens, scale,
                   softcap, lam, norm_eps, out_mult, out_dtype, head_bias=None,
                   gate=None, shared_kv=False, out_rot_cs=None,
-                  out_rot_interleaved=False, value_col=0):
+                  out_rot_interleaved=False, value_col=0, dist_bias=None,
+                  sink=None):
     """Attention over cache rows [keys (kv_heads x maps x dim) |
     values (kv_heads x vdim)]; shared_kv: a row holds the keys only (one kv
     head, one map) and the values are its columns value_col .. value_col +
@@ -865,7 +873,11 @@ def row_attention(q, cache, pool, block_tables, token_seq, positions, heads,
     the head's result is divided by its RMS and multiplied by out_mult.
     head_bias [heads] given: no softmax; a visible key weighs sigmoid(s +
     head_bias[h]) and the weights are not normalised over the keys. gate
-    [T, heads] given: head h's result is multiplied by sigmoid(gate[t, h]).
+    [T, heads] given: head h's result is multiplied by sigmoid(gate[t, h]);
+    gate [T, heads * vdim]: element by element. dist_bias [heads, N] given: a
+    key n positions back gets dist_bias[h, min(n, N - 1)] added to its scaled
+    score. sink [heads] given: the softmax's denominator also holds
+    exp(sink[h]).
     out_rot_cs [T, vdim / 2, 2] (cos, sin per token and pair) given: every
     head's result is turned BACK by its token's angles over the whole value
     width (pair m = dimensions m, m + vdim / 2, or 2m, 2m + 1 when
@@ -897,8 +909,14 @@ def row_attention(q, cache, pool, block_tables, token_seq, positions, heads,
         s = torch.einsum("grmd,ngmd->grmn", qv[t], k) * scale
         if softcap > 0:
             s = softcap * torch.tanh(s / softcap)
+        if dist_bias is not None:
+            n = (p - j).clamp(max=dist_bias.shape[1] - 1)
+            s = s + dist_bias.float()[:, n].view(G, rep, 1, -1)
         if head_bias is not None:
             wts = torch.sigmoid(s + head_bias.float().view(G, rep, 1, 1))
+        elif sink is not None:   # a key-less term of the denominator
+            s = torch.cat([s, sink.float().view(G, rep, 1, 1).expand(G, rep, M, 1)], -1)
+            wts = torch.softmax(s, dim=-1)[..., :-1]
         else:
             wts = torch.softmax(s, dim=-1)
         a = torch.einsum("grmn,ngv->grmv", wts, v)
@@ -906,7 +924,7 @@ def row_attention(q, cache, pool, block_tables, token_seq, positions, heads,
         if norm_eps is not None:
             o = o / torch.sqrt((o * o).mean(-1, keepdim=True) + norm_eps) * out_mult
         if gate is not None:
-            o = o * torch.sigmoid(gate[t].float()).view(G, rep, 1)
+            o = o * torch.sigmoid(gate[t].float()).view(G, rep, -1)
         out[t] = o.reshape(H, vdim)
     if out_rot_cs is not None:
         cs = out_rot_cs.view(T, 1, vdim // 2, 2).float()
@@ -1132,17 +1150,31 @@ def linear_f32(x, weight):
     return x.float() @ weight.float().t()
 
 
-def route_softmax(x, weight, bias, experts, top):
+def route_softmax(x, weight, bias, experts, top, groups=1, keep=1):
     """Router over the first `experts` rows of weight [N, W], N >= experts:
     the `top` largest of z = x W^T + bias, weights = softmax over those; the
-    rows after the experts are plain fp32 outputs. Returns (ids [T, top]
+    rows after the experts are plain fp32 outputs. groups > 1: the experts
+    form `groups` equal runs of neighbours and only those of the `keep` runs
+    with the largest single logit can be chosen. Returns (ids [T, top]
     int64, weights [T, top] fp32, rest [T, N - experts] fp32)."""
     z = linear_f32(x, weight)
     zr = z[:, :experts]
     if bias is not None:
         zr = zr + bias.float()
-    val, ids = zr.topk(top, dim=-1)
+    val, ids = limit_to_groups(zr, groups, keep).topk(top, dim=-1)
     return ids, torch.softmax(val, dim=-1), z[:, experts:].contiguous()
+
+
+def limit_to_groups(z, groups, keep):
+    """z [T, E] with -inf outside the `keep` of `groups` equal runs of columns
+    whose largest entry is largest."""
+    if groups <= 1 or keep >= groups:
+        return z
+    v = z.view(z.shape[0], groups, -1)
+    best = v.amax(-1).topk(keep, dim=-1).indices
+    off = torch.ones(v.shape[:2], dtype=torch.bool, device=z.device)
+    off.scatter_(1, best, False)
+    return v.masked_fill(off.unsqueeze(-1), float("-inf")).view_as(z)
 
 
 def biased_glu(gate_up, bias, act):
@@ -1162,3 +1194,142 @@ def softcap_logits(x, scale, cap):
     """fp32: z = x * scale; cap > 0: cap * tanh(z / cap)."""
     z = x.float() * scale
     return cap * torch.tanh(z / cap) if cap > 0 else z
+
+
+# -- parallel layers with two norms, short convolution, decaying linear attention,
+# gated delta rule ------------------------------------------------------------------
+
+
+def parallel_rmsnorm_add(x, a, b, wa, wb, scale, f, w1, w2, eps, offset, out_dtype):
+    """One step of a residual stream whose mixer and feed-forward run side by
+    side, each on a norm of its own. x [T, W] fp32, in place:
+      m = a                                              (b None)
+        = scale * (a / rms(a) * wa + b / rms(b) * wb)    (two mixers)
+      x <- x + (m + f)           (a None, f None: without that part)
+      h_i = x / rms(x) * (offset + w_i)
+    rms(v) = sqrt(mean(v^2) + eps). Returns (h1, h2) in out_dtype, None where
+    w_i is None."""
+    def unit(v):
+        return v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps)
+
+    add = None
+    if a is not None:
+        add = a.float()
+        if b is not None:
+            add = scale * (unit(add) * wa.float() + unit(b.float()) * wb.float())
+    if f is not None:
+        add = f.float() if add is None else add + f.float()
+    if add is not None:
+        x.add_(add)
+    n = unit(x)
+    return tuple((n * (offset + w.float())).to(out_dtype) if w is not None else None
+                 for w in (w1, w2))
+
+
+def short_conv(x, weight, state, slots, cu, positions, out_dtype):
+    """Causal depthwise convolution over packed sequences, then silu. x [T, C],
+    weight [C, taps] (last column: the current token's), state [slots, C, taps
+    - 1] holds the inputs before the portion (read as zeros when it begins at
+    position 0) and receives the last ones. Returns [T, C]."""
+    T, C = x.shape
+    n = weight.shape[1] - 1
+    w = weight.float()
+    out = torch.empty(T, C, dtype=torch.float32)
+    bounds = cu.tolist() if cu is not None else list(range(T + 1))
+    pos = positions.tolist()
+    for b, slot in enumerate(slots.tolist()):
+        t0, t1 = bounds[b], bounds[b + 1]
+        if t0 >= t1:
+            continue
+        past = state[slot].float()
+        if pos[t0] == 0:
+            past = torch.zeros_like(past)
+        full = torch.cat([past, x[t0:t1].float().t()], dim=-1)     # [C, n + L]
+        win = full.unfold(-1, n + 1, 1)                            # [C, L, taps]
+        out[t0:t1] = (win * w.unsqueeze(1)).sum(-1).t()
+        state[slot] = full[:, full.shape[1] - n:].to(state.dtype)
+    return torch.nn.functional.silu(out).to(out_dtype)
+
+
+def rope_table(positions, freq):
+    """fp32 [T, 2 n]: (cos, sin) of pos * freq[i], pairs side by side."""
+    ang = positions.float().unsqueeze(-1) * freq.float()
+    return torch.stack([torch.cos(ang), torch.sin(ang)], -1).flatten(1)
+
+
+def _rotate_by_table(x, cs):
+    """x [T, H, d] fp32: pair (i, i + n) of every head by the token's n (cos,
+    sin) pairs; the dimensions from 2 n on pass."""
+    n = cs.shape[1] // 2
+    c, s = cs[:, 0::2].unsqueeze(1), cs[:, 1::2].unsqueeze(1)
+    u, v = x[..., :n], x[..., n : 2 * n]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * n :]], -1)
+
+
+def decay_attention(q, k, v, decay, k_scale, silu, rot_cs, state, slots, cu,
+                    positions):
+    """Linear attention with a fixed decay per head over packed sequences. q, k
+    [T, H, d], v [T, H, dv] as projected; silu: q, k and v pass silu first;
+    rot_cs [T, 2 n]: q and k are rotated (pairs i, i + n); k is multiplied by
+    k_scale. S_t = decay_h S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, all fp32; the
+    state [slots, H, d, dv] is read (or started from zero at position 0) and
+    written back. Returns fp32 [T, H, dv]."""
+    qf, kf, vf = q.float(), k.float(), v.float()
+    if silu:
+        qf, kf, vf = (torch.nn.functional.silu(t) for t in (qf, kf, vf))
+    if rot_cs is not None:
+        qf, kf = _rotate_by_table(qf, rot_cs), _rotate_by_table(kf, rot_cs)
+    kf = kf * k_scale
+    T, H, _ = q.shape
+    dec = decay.float().view(H, 1, 1)
+    o = torch.empty(T, H, v.shape[2], dtype=torch.float32)
+    bounds = cu.tolist() if cu is not None else list(range(T + 1))
+    pos = positions.tolist()
+    for b, slot in enumerate(slots.tolist()):
+        t0, t1 = bounds[b], bounds[b + 1]
+        if t0 >= t1:
+            continue
+        S = torch.zeros_like(state[slot]) if pos[t0] == 0 else state[slot].clone()
+        for t in range(t0, t1):
+            S = dec * S + kf[t].unsqueeze(-1) * vf[t].unsqueeze(-2)
+            o[t] = torch.einsum("hkv,hk->hv", S, qf[t])
+        state[slot] = S
+    return o
+
+
+def gated_delta_rule(q, k, v, gates, a_log, dt_bias, state, slots, cu, positions):
+    """Gated delta rule over packed sequences. q, k [T, G, d], v [T, H, dv]
+    (head h reads q/k head h // (H / G)); gates [T, 2 H] = [step size | decay]
+    pre-activations. q, k are made unit vectors (eps 1e-6 under the root), q
+    is multiplied by d^-1/2; beta = sigmoid(.), g = exp(-exp(a_log)
+    softplus(. + dt_bias)). Per head S <- g S, u = beta (v - S^T k), S <- S +
+    k u^T, o = S^T q, all fp32; state as in decay_attention. Returns fp32
+    [T, H, dv]."""
+    T, G, d = q.shape
+    H = v.shape[1]
+
+    def unit(x):
+        x = x.float()
+        return (x / torch.sqrt((x * x).sum(-1, keepdim=True) + 1e-6)) \
+            .repeat_interleave(H // G, dim=1)
+
+    qf, kf, vf = unit(q) * d ** -0.5, unit(k), v.float()
+    z = gates.float()
+    beta = torch.sigmoid(z[:, :H])
+    dec = torch.exp(-torch.exp(a_log.float())
+                    * torch.nn.functional.softplus(z[:, H:] + dt_bias.float()))
+    o = torch.empty(T, H, v.shape[2], dtype=torch.float32)
+    bounds = cu.tolist() if cu is not None else list(range(T + 1))
+    pos = positions.tolist()
+    for b, slot in enumerate(slots.tolist()):
+        t0, t1 = bounds[b], bounds[b + 1]
+        if t0 >= t1:
+            continue
+        S = torch.zeros_like(state[slot]) if pos[t0] == 0 else state[slot].clone()
+        for t in range(t0, t1):
+            S = dec[t].view(H, 1, 1) * S
+            u = beta[t].view(H, 1) * (vf[t] - torch.einsum("hkv,hk->hv", S, kf[t]))
+            S = S + kf[t].unsqueeze(-1) * u.unsqueeze(-2)
+            o[t] = torch.einsum("hkv,hk->hv", S, qf[t])
+        state[slot] = S
+    return o

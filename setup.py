@@ -6,7 +6,8 @@ The built .so files land at parallax_amd/ops/_C.*.so (attention, GEMM, MoE,
 sampler kernels) and parallax_amd/ops/_mix.*.so (sequence mixers: fp32-residual
 layer norm, sliding-window latent attention, gated linear attention, sandwich
 RMS norm, row-cache attention, post-norm residual step, minGRU, hyper-connected
-streams, matrix LSTM, softmax router). Both are
+streams, matrix LSTM, softmax router, fixed-decay linear attention, gated delta
+rule, short convolution). Both are
 git-ignored; they travel to the GPU box with the gpurun snapshot.
 PARALLAX_EXT=_mix (or _C) builds one of them only.
 """
@@ -60,6 +61,8 @@ mix_sources = [
     os.path.join(CSRC, "hyper.hip"),
     os.path.join(CSRC, "small_linear.hip"),
     os.path.join(CSRC, "mlstm.hip"),
+    os.path.join(CSRC, "linear_recurrence.hip"),
+    os.path.join(CSRC, "short_conv.hip"),
 ]
 
 wanted = [x for x in os.environ.get("PARALLAX_EXT", "_C,_mix").split(",") if x]
