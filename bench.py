@@ -409,6 +409,56 @@ def vurizen_like_config(z: dict) -> dict:
     return cfg
 
 
+# `--design-compare --design-pair domelix`: a Domelix stack (softmax attention
+# with a distance bias beside lightning attention, gated delta rule, retention,
+# routed experts beside the mixer) beside a Runidra stack of EQUAL sizes (matrix
+# LSTM layers where this one has a delta rule or retention, latent attention
+# layers where it has the parallel mixer; the same head widths, heads and
+# experts, one residual stream, no loop, no shared expert, a window as long as
+# the context).
+
+DOMELIX_SIZES = {
+    "s": dict(width=1024, layers=8, heads=8, kv_heads=2, dim=64, experts=16, top=2,
+              ff=512, groups=4, keep=2, vocab=32000),
+    "m": dict(width=2048, layers=8, heads=16, kv_heads=4, dim=128, experts=32, top=4,
+              ff=1024, groups=4, keep=2, vocab=32000),
+    "l": dict(width=4096, layers=8, heads=32, kv_heads=8, dim=128, experts=32, top=4,
+              ff=1024, groups=4, keep=2, vocab=32000),
+}
+_DOMELIX_ORDER = ("retention", "parallel", "delta", "parallel")
+
+
+def domelix_config(z: dict) -> dict:
+    mlp = {"kind": "moe", "expert": {"ff": z["ff"]},
+           "router": {"experts": z["experts"], "top": z["top"],
+                      "groups": {"count": z["groups"], "keep": z["keep"]}}}
+    H, d = z["heads"], z["dim"]
+    decay = [1.0 - 2.0 ** (-5.0 - 7.0 * i / max(1, H - 1)) for i in range(H)]
+    mixers = {
+        "retention": {"heads": H, "dim": d, "vdim": d, "decay": decay,
+                      "rot": {"base": 10000.0, "dims": d}},
+        "parallel": {"left": {"heads": H, "kv_heads": z["kv_heads"], "dim": d, "vdim": d,
+                              "scale": d ** -0.5, "bias_max": 128},
+                     "right": {"heads": H // 2, "dim": d, "vdim": d,
+                               "decay": decay[: H // 2]}},
+        "delta": {"heads": H, "kv_heads": H // 2, "dim": d, "vdim": d, "conv": 4},
+    }
+    order = [_DOMELIX_ORDER[i % 4] for i in range(z["layers"])]
+    return {"architecture": "Domelix",
+            "layers": [{"type": k, "mixer": mixers[k], "mlp": mlp} for k in order],
+            "norm": {"eps": 1e-5}, "vocab": z["vocab"], "width": z["width"]}
+
+
+def runidra_like_domelix_config(z: dict) -> dict:
+    cfg = runidra_config(dict(
+        z, nope=z["dim"], rot=64, vdim=z["dim"], rank=512, q_rank=z["width"] // 2,
+        window=1 << 20, streams=1))
+    cell, latent = cfg["layers"][0], cfg["layers"][1]
+    cfg["layers"] = [latent if _DOMELIX_ORDER[i % 4] == "parallel" else cell
+                     for i in range(z["layers"])]
+    return cfg
+
+
 def design_compare(args) -> None:
     from parallax_amd.models.config import ModelConfig
     from parallax_amd.server.engine import Engine, EngineArgs
@@ -432,6 +482,10 @@ def design_compare(args) -> None:
             z = RUNIDRA_SIZES[size]
             pair = (("runidra", runidra_config(z)),
                     ("vurizen-like", vurizen_like_config(z)))
+        elif args.design_pair == "domelix":
+            z = DOMELIX_SIZES[size]
+            pair = (("domelix", domelix_config(z)),
+                    ("runidra-like", runidra_like_domelix_config(z)))
         else:
             z = DESIGN_SIZES[size]
             pair = (("vurizen", vurizen_config(z)),
@@ -540,22 +594,24 @@ def main():
                          "throughput of a Vurizen stack beside a DeepSeek-V3-"
                          "style stack of equal sizes (one GPU, random weights)")
     ap.add_argument("--design-pair", default="vurizen",
-                    choices=["vurizen", "sogidra", "zabusun", "pudizen", "runidra"],
+                    choices=["vurizen", "sogidra", "zabusun", "pudizen", "runidra",
+                             "domelix"],
                     help="which design --design-compare measures: vurizen "
                          "beside a DeepSeek-V3-style stack, sogidra beside "
                          "a Qwen3-style dense stack, zabusun beside a "
                          "Qwen3-MoE-style stack, pudizen beside a "
-                         "Qwen3-style dense stack, or runidra beside a "
-                         "vurizen stack")
+                         "Qwen3-style dense stack, runidra beside a "
+                         "vurizen stack, or domelix beside a runidra stack")
     ap.add_argument("--design-sizes", default="s,m",
                     help="comma list of " + ",".join(DESIGN_SIZES)
-                    + " (the pudizen and runidra pairs also have l)")
+                    + " (the pudizen, runidra and domelix pairs also have l)")
     ap.add_argument("--design-batch", type=int, default=8)
     ap.add_argument("--design-prompt", type=int, default=2048)
     ap.add_argument("--design-only", default="",
                     help="one design of the pair (vurizen | deepseek-like | "
                          "sogidra | qwen3-like | zabusun | qwen3-moe-like | "
-                         "pudizen | runidra | vurizen-like; "
+                         "pudizen | runidra | vurizen-like | domelix | "
+                         "runidra-like; "
                          "default: both)")
     args = ap.parse_args()
     if args.design_compare:
