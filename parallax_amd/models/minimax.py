@@ -10,20 +10,19 @@ a Mixtral-style softmax top-k MoE, and the residual stream is the MiniMax
 norm-first variant: residual = NORMED hidden, combined with configurable
 alpha/beta factors.
 
-Prefill replicates the HF 256-token block recursion exactly (intra-block
-decay matrix + inter-block decayed state), so chunked prefill at any boundary
-is bit-consistent with a single-shot prefill; decode is one batched recurrence
-step (graph-capturable einsums over the slot-indexed state)."""
+The recurrence is ops.decay_attention, which the fixed-decay mixer of
+linear_attention.py uses too: prompt portions run in chunks continued from the
+cached state (HIP kernels; a portion may end anywhere), decode is one batched,
+graph-capturable step; norm over all heads and sigmoid gate are one kernel
+(ops.gated_rmsnorm)."""
 
 from __future__ import annotations
 
 import math
-from typing import Optional
-
 import torch
 import torch.nn as nn
-import torch.nn.functional as F
 
+from .. import ops
 from .config import ModelConfig
 from .forward_meta import ForwardMeta
 from .llama import LlamaAttention, LlamaShardModel, RMSNorm
@@ -37,7 +36,6 @@ class LightningAttention(nn.Module):
         self.linear_layer_idx = linear_layer_idx
         self.num_heads = cfg.num_heads
         self.head_dim = cfg.head_dim
-        self.block_size = int(cfg.raw.get("block_size", 256))
         h = cfg.hidden_size
         H, d = self.num_heads, self.head_dim
         self.qkv_proj = nn.Linear(h, 3 * H * d, bias=False)
@@ -48,75 +46,23 @@ class LightningAttention(nn.Module):
         # HF get_slope_rate) — recomputed here, the HF buffers are ignored
         base = 1.0 / (2.0 ** (8.0 / H))
         factor = 1.0 - layer_idx / (cfg.num_layers - 1 + 1e-5) + 1e-5
-        slope = torch.tensor(
-            [base ** (i + 1) * factor for i in range(H)], dtype=torch.float32
-        )
-        self.register_buffer("slope_rate", slope, persistent=False)
+        self._powers = ops.decay_powers(
+            [math.exp(-(base ** (i + 1)) * factor) for i in range(H)])
 
     def forward(self, x: torch.Tensor, meta: ForwardMeta, rope_cache) -> torch.Tensor:
         T = x.shape[0]
         H, d = self.num_heads, self.head_dim
-        qkv = F.silu(self.qkv_proj(x)).view(T, H, 3 * d)
+        qkv = self.qkv_proj(x).view(T, H, 3 * d)
         q, k, v = torch.split(qkv, [d, d, d], dim=-1)
-        rec = meta.linear_cache.recurrent_states[self.linear_layer_idx]
-        slots = meta.linear_slots
-        if meta.is_prefill:
-            core = self._prefill(q, k, v, meta, rec, slots)
-        else:
-            core = self._decode(q, k, v, rec, slots)
-        out = self.norm(core.reshape(T, H * d).to(x.dtype))
-        out = torch.sigmoid(self.output_gate(x).float()).to(out.dtype) * out
-        return self.out_proj(out)
-
-    def _decode(self, q, k, v, rec, slots):
-        """One recurrence step for all sequences: S <- ratio*S + k^T v;
-        out = q S. Batched einsums, hipGraph-capturable."""
-        S = rec[slots]                                   # [B, H, d, d] fp32
-        qf, kf, vf = q.float(), k.float(), v.float()
-        ratio = torch.exp(-self.slope_rate).view(1, -1, 1, 1)
-        S = S * ratio + torch.einsum("bhk,bhv->bhkv", kf, vf)
-        out = torch.einsum("bhk,bhkv->bhv", qf, S)
-        rec[slots] = S
-        return out.to(q.dtype)
-
-    def _prefill(self, q, k, v, meta: ForwardMeta, rec, slots):
-        """HF block recursion (block_size tokens at a time) continued from the
-        cached state, so chunk boundaries do not change the math."""
-        B = self.block_size
-        sr = self.slope_rate.view(-1, 1, 1)              # [H,1,1]
-        outs = []
-        t0 = 0
-        for i in range(meta.batch_size):
-            L = int(meta.query_lens[i])
-            slot = int(slots[i])
-            S = rec[slot].clone()                        # [H, d, d] fp32
-            qf = q[t0:t0 + L].float().transpose(0, 1)    # [H, L, d]
-            kf = k[t0:t0 + L].float().transpose(0, 1)
-            vf = v[t0:t0 + L].float().transpose(0, 1)
-            out = torch.empty_like(qf)
-            for s0 in range(0, L, B):
-                e = min(s0 + B, L)
-                n = e - s0
-                r = torch.arange(n, dtype=torch.float32, device=q.device)
-                qb, kb, vb = qf[:, s0:e], kf[:, s0:e], vf[:, s0:e]
-                # intra-block: (Q K^T ∘ exp(-slope (i-j)), i>=j) V
-                diag = (r.view(1, -1, 1) - r.view(1, 1, -1)) * sr
-                diag = torch.where(diag >= 0, torch.exp(-diag),
-                                   torch.zeros_like(diag))
-                intra = torch.matmul(torch.matmul(qb, kb.transpose(-1, -2)) * diag, vb)
-                # inter-block: decayed query against the carried state
-                qdec = torch.exp(-sr * (r.view(1, -1, 1) + 1.0))
-                inter = torch.matmul(qb * qdec, S)
-                out[:, s0:e] = inter + intra
-                # fold this block into the state
-                kdec = torch.exp(-sr * (n - 1 - r).view(1, -1, 1))
-                S = S * torch.exp(-sr * n) + torch.matmul(
-                    (kb * kdec).transpose(-1, -2), vb
-                )
-            rec[slot] = S
-            outs.append(out.transpose(0, 1).to(q.dtype))
-            t0 += L
-        return torch.cat(outs, dim=0)
+        if self._powers.device != x.device:
+            self._powers = self._powers.to(x.device)
+        core = ops.decay_attention(
+            q, k, v, self._powers, 1.0, True, None,
+            meta.linear_cache.recurrent_states[self.linear_layer_idx],
+            meta.linear_slots, meta.query_bounds(), meta.positions)
+        return self.out_proj(ops.gated_rmsnorm(
+            core, self.output_gate(x), self.norm.weight, self.norm.eps, x.dtype,
+            whole=True, act="sigmoid"))
 
 
 class MiniMaxMoE(nn.Module):

@@ -5,19 +5,16 @@ shared expert.
 Reference analogue: src/parallax/models/qwen3_next.py (hybrid linear+full
 attention with conv/recurrent state slots, cache/linear_cache.py). Fresh
 design: state lives in LinearStateCache slots (conv window + fp32 recurrent
-state per request); decode is a fully batched single-step recurrence
-(graph-capturable), prefill is a per-request scan. A fused HIP step kernel is a
-later optimization — the per-token recurrence math is tiny next to the MoE.
+state per request); the convolution, the recurrence and the gated norm are the
+ops that the delta-rule mixer of linear_attention.py uses too (ops.short_conv,
+ops.gated_delta_rule, ops.gated_rmsnorm: HIP kernels for prompt portions, in
+chunks, and for batched decode steps).
 """
 
 from __future__ import annotations
 
-import math
-from typing import Optional
-
 import torch
 import torch.nn as nn
-import torch.nn.functional as F
 
 from .. import ops
 from ..parallel.layers import MergedColumnParallelLinear
@@ -28,23 +25,14 @@ from .moe import FusedMoE
 from .registry import register_model
 
 
-def _l2norm(x: torch.Tensor, eps: float = 1e-6) -> torch.Tensor:
-    return x * torch.rsqrt((x.float() ** 2).sum(-1, keepdim=True) + eps).to(x.dtype)
-
-
 class GatedRMSNorm(nn.Module):
-    """RMSNorm then multiply by silu(gate) (HF Qwen3NextRMSNormGated)."""
+    """The weight of an RMSNorm that is followed by silu(gate) (HF
+    Qwen3NextRMSNormGated); ops.gated_rmsnorm does the work."""
 
     def __init__(self, dim: int, eps: float):
         super().__init__()
         self.weight = nn.Parameter(torch.empty(dim), requires_grad=False)
         self.eps = eps
-
-    def forward(self, x: torch.Tensor, gate: torch.Tensor) -> torch.Tensor:
-        xf = x.float()
-        xf = xf * torch.rsqrt(xf.pow(2).mean(-1, keepdim=True) + self.eps)
-        xf = xf * self.weight.float()
-        return (xf * F.silu(gate.float())).to(x.dtype)
 
 
 class GatedDeltaNet(nn.Module):
@@ -99,111 +87,21 @@ class GatedDeltaNet(nn.Module):
             [q.reshape(T, -1), k.reshape(T, -1), v.reshape(T, -1)], dim=-1
         )  # [T, conv_dim]
 
-        conv_states = meta.linear_cache.conv_states[self.linear_layer_idx]
-        rec_states = meta.linear_cache.recurrent_states[self.linear_layer_idx]
-        slots = meta.linear_slots
-
-        if meta.is_prefill:
-            mixed = self._conv_prefill(mixed, meta, conv_states, slots)
-        else:
-            mixed = self._conv_decode(mixed, conv_states, slots)
-
+        idx, cu = self.linear_layer_idx, meta.query_bounds()
+        cache, slots = meta.linear_cache, meta.linear_slots
+        mixed = ops.short_conv(mixed, self.conv_weight, cache.conv_states[idx],
+                               slots, cu, meta.positions, x.dtype)
         q, k, v = torch.split(
             mixed, [self.key_dim, self.key_dim, self.value_dim], dim=-1
         )
-        q = _l2norm(q.view(T, self.hk, self.dk))
-        k = _l2norm(k.view(T, self.hk, self.dk))
-        v = v.view(T, self.hv, self.dv)
-        g_ratio = self.hv // self.hk
-        if g_ratio > 1:
-            q = q.repeat_interleave(g_ratio, dim=1)
-            k = k.repeat_interleave(g_ratio, dim=1)
-
-        beta = b.float().sigmoid()                                   # [T, Hv]
-        gdecay = -self.A_log.float().exp() * F.softplus(a.float() + self.dt_bias.float())
-        scale = self.dk ** -0.5
-
-        if meta.is_prefill:
-            core = self._delta_prefill(q, k, v, gdecay, beta, scale, meta,
-                                       rec_states, slots)
-        else:
-            core = self._delta_decode(q, k, v, gdecay, beta, scale,
-                                      rec_states, slots)
-
-        out = self.norm(core.reshape(T * self.hv, self.dv),
-                        z.reshape(T * self.hv, self.dv))
-        return self.out_proj(out.view(T, self.value_dim))
-
-    # -- causal conv front-end ---------------------------------------------------
-
-    def _conv_decode(self, mixed, conv_states, slots):
-        """Batched single-token conv window update (graph-capturable)."""
-        state = conv_states[slots]                       # [B, conv_dim, K-1]
-        window = torch.cat([state.to(mixed.dtype), mixed.unsqueeze(-1)], dim=-1)
-        out = (window.float() * self.conv_weight.float()).sum(-1)
-        conv_states[slots] = window[..., 1:].to(conv_states.dtype)
-        return F.silu(out).to(mixed.dtype)
-
-    def _conv_prefill(self, mixed, meta: ForwardMeta, conv_states, slots):
-        outs = []
-        t0 = 0
-        for i in range(meta.batch_size):
-            L = int(meta.query_lens[i])
-            slot = int(slots[i])
-            seq = mixed[t0 : t0 + L].T                  # [conv_dim, L]
-            state = conv_states[slot].to(seq.dtype)     # [conv_dim, K-1]
-            padded = torch.cat([state, seq], dim=-1)    # [conv_dim, K-1+L]
-            out = F.conv1d(
-                padded.float().unsqueeze(0),
-                self.conv_weight.float().unsqueeze(1),
-                groups=self.conv_dim,
-            )[0]                                         # [conv_dim, L]
-            conv_states[slot] = padded[:, -(self.kernel - 1):].to(conv_states.dtype)
-            outs.append(F.silu(out).T.to(mixed.dtype))
-            t0 += L
-        return torch.cat(outs, dim=0)
-
-    # -- gated delta rule ------------------------------------------------------------
-
-    def _delta_decode(self, q, k, v, g, beta, scale, rec_states, slots):
-        """One recurrence step for every sequence at once.
-        S <- S * exp(g);  out_mem = k^T S;  delta = beta (v - out_mem);
-        S <- S + k^T delta;  out = (q*scale)^T S   (per head)."""
-        S = rec_states[slots].float()                    # [B, Hv, dk, dv]
-        qf, kf, vf = q.float(), k.float(), v.float()
-        S = S * g.exp().unsqueeze(-1).unsqueeze(-1)
-        kv_mem = torch.einsum("bhk,bhkv->bhv", kf, S)
-        delta = (vf - kv_mem) * beta.unsqueeze(-1)
-        S = S + torch.einsum("bhk,bhv->bhkv", kf, delta)
-        out = torch.einsum("bhk,bhkv->bhv", qf * scale, S)
-        rec_states[slots] = S
-        return out.to(q.dtype)
-
-    def _delta_prefill(self, q, k, v, g, beta, scale, meta: ForwardMeta,
-                       rec_states, slots):
-        outs = []
-        t0 = 0
-        for i in range(meta.batch_size):
-            L = int(meta.query_lens[i])
-            slot = int(slots[i])
-            S = rec_states[slot].float()                 # [Hv, dk, dv]
-            qf = q[t0 : t0 + L].float() * scale
-            kf = k[t0 : t0 + L].float()
-            vf = v[t0 : t0 + L].float()
-            gf = g[t0 : t0 + L].exp()
-            bf = beta[t0 : t0 + L]
-            out = torch.empty(L, self.hv, self.dv, dtype=torch.float32,
-                              device=q.device)
-            for t in range(L):
-                S = S * gf[t].unsqueeze(-1).unsqueeze(-1)
-                kv_mem = torch.einsum("hk,hkv->hv", kf[t], S)
-                delta = (vf[t] - kv_mem) * bf[t].unsqueeze(-1)
-                S = S + torch.einsum("hk,hv->hkv", kf[t], delta)
-                out[t] = torch.einsum("hk,hkv->hv", qf[t], S)
-            rec_states[slot] = S
-            outs.append(out.to(q.dtype))
-            t0 += L
-        return torch.cat(outs, dim=0)
+        core = ops.gated_delta_rule(
+            q.view(T, self.hk, self.dk), k.view(T, self.hk, self.dk),
+            v.view(T, self.hv, self.dv), torch.cat([b, a], dim=-1).float(),
+            self.A_log.float(), self.dt_bias.float(),
+            cache.recurrent_states[idx], slots, cu, meta.positions)
+        out = ops.gated_rmsnorm(core, z.reshape(T, self.value_dim),
+                                self.norm.weight, self.norm.eps, x.dtype)
+        return self.out_proj(out)
 
 
 class Qwen3NextAttention(LlamaAttention):

@@ -561,9 +561,14 @@ __global__ __launch_bounds__(256) void row_attention_kernel(
     const bool valid = u < nk;
     int64_t off = 0;
     bool pooled = false;
-    float s[NQ];
+    float s[NQ], bv[NQ];
 #pragma unroll
-    for (int n = 0; n < NQ; ++n) s[n] = 0.f;
+    for (int n = 0; n < NQ; ++n) {
+      s[n] = bv[n] = 0.f;
+      if (dist_bias != nullptr && valid)   // no pooled rows: key u is lo + u
+        bv[n] = dist_bias[(int64_t)(g * rep + min(r0 + n / M, rep - 1)) * n_bias +
+                          min(pos - lo - u, n_bias - 1)];
+    }
     if (valid) {
       pooled = POOL && u < nb;
       if (pooled) {
@@ -599,9 +604,7 @@ __global__ __launch_bounds__(256) void row_attention_kernel(
     for (int n = 0; n < NQ; ++n) {
       float sc = s[n] * scale;
       if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
-      if (dist_bias != nullptr && valid)   // no pooled rows: key u is lo + u
-        sc += dist_bias[(int64_t)(g * rep + min(r0 + n / M, rep - 1)) * n_bias +
-                        min(pos - lo - u, n_bias - 1)];
+      sc += bv[n];
       float p;
       if (sig) {
         p = valid ? ra_sigmoid(sc + hb[n]) : 0.f;

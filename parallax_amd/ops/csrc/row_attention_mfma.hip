@@ -104,6 +104,10 @@ DEVINL float rm_tanh(float x) {
   return 1.0f - 2.0f * __frcp_rn(__expf(2.0f * x) + 1.0f);
 }
 
+#define RM_LOG2E 1.44269504088896340736f
+// 2^x, the hardware's
+DEVINL float rm_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
+
 // sigmoid through the same two hardware approximations
 DEVINL float rm_sigmoid(float x) { return __frcp_rn(1.0f + __expf(-x)); }
 // outside the inner loops: the library exponential
@@ -651,10 +655,12 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_bf16_kernel(
   float mx = -INFINITY, l = 0.f;
   const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
   const float hbias = SIG ? head_bias[h] : 0.f;
+  // softmax scores are kept times log2(e), so that a weight is one 2^x
+  const float scale2 = scale * RM_LOG2E, cap2 = softcap * RM_LOG2E;
   const float* brow = (REL && dist_bias) ? dist_bias + (int64_t)h * n_bias : nullptr;
-  const float bfar = brow ? brow[n_bias - 1] : 0.f;
+  const float bfar = brow ? brow[n_bias - 1] * RM_LOG2E : 0.f;
   if (REL && sink) {
-    mx = sink[h];
+    mx = sink[h] * RM_LOG2E;
     l = 1.f;
   }
 
@@ -733,35 +739,54 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_bf16_kernel(
     float corr = 1.f;
     if (SIG) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
+      for (int i = 0; i < 16; ++i) {
+        float sc = S[i] * scale;
+        if (softcap > 0.f) sc = softcap * rm_tanh(sc * inv_cap);
+        S[i] = rm_sigmoid(sc + hbias);
+      }
+      if (!interior) {
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int u = u0 + 8 * i + 4 * half + j;
+        for (int i = 0; i < 16; ++i) {
+          const int u = u0 + 8 * (i >> 2) + 4 * half + (i & 3);
           const int jt = lo + u;
-          const bool vis = interior || (jt <= pq && (window == 0 || pq - jt < window) &&
-                                        qvalid && u < nk);
-          float sc = S[4 * i + j] * scale;
-          if (softcap > 0.f) sc = softcap * rm_tanh(sc * inv_cap);
-          S[4 * i + j] = vis ? rm_sigmoid(sc + hbias) : 0.f;
+          const bool vis = jt <= pq && (window == 0 || pq - jt < window) && qvalid &&
+                           u < nk;
+          S[i] = vis ? S[i] : 0.f;
         }
+      }
     } else {
       float tmax = -INFINITY;
-      const bool far = REL && p0 - (jt0 + RM_K - 1) >= n_bias - 1;
+      if (softcap > 0.f) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
+        for (int i = 0; i < 16; ++i) S[i] = cap2 * rm_tanh(S[i] * scale * inv_cap);
+      } else {
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int u = u0 + 8 * i + 4 * half + j;
-          const int jt = lo + u;
-          const bool vis = interior || (jt <= pq && (window == 0 || pq - jt < window) &&
-                                        qvalid && u < nk);
-          float sc = S[4 * i + j] * scale;
-          if (softcap > 0.f) sc = softcap * rm_tanh(sc * inv_cap);
-          if (REL && brow) sc += far ? bfar : brow[min(max(pq - jt, 0), n_bias - 1)];
-          sc = vis ? sc : -INFINITY;
-          S[4 * i + j] = sc;
-          tmax = fmaxf(tmax, sc);
+        for (int i = 0; i < 16; ++i) S[i] *= scale2;
+      }
+      if (REL && brow) {
+        if (p0 - (jt0 + RM_K - 1) >= n_bias - 1) {
+#pragma unroll
+          for (int i = 0; i < 16; ++i) S[i] += bfar;
+        } else {
+#pragma unroll
+          for (int i = 0; i < 16; ++i) {
+            const int jt = jt0 + 8 * (i >> 2) + 4 * half + (i & 3);
+            S[i] = fmaf(brow[min(max(pq - jt, 0), n_bias - 1)], RM_LOG2E, S[i]);
+          }
         }
+      }
+      if (!interior) {
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+          const int u = u0 + 8 * (i >> 2) + 4 * half + (i & 3);
+          const int jt = lo + u;
+          const bool vis = jt <= pq && (window == 0 || pq - jt < window) && qvalid &&
+                           u < nk;
+          S[i] = vis ? S[i] : -INFINITY;
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < 16; ++i) tmax = fmaxf(tmax, S[i]);
       tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
       const float m_new = fmaxf(mx, tmax);
       float psum = 0.f;
@@ -769,10 +794,10 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_bf16_kernel(
 #pragma unroll
         for (int i = 0; i < 16; ++i) S[i] = 0.f;
       } else {
-        corr = __expf(mx - m_new);  // exp(-inf) = 0 the first time a key is seen
+        corr = rm_exp2(mx - m_new);  // 2^-inf = 0 the first time a key is seen
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
-          const float p = __expf(S[i] - m_new);  // exp(-inf) = 0 for masked keys
+          const float p = rm_exp2(S[i] - m_new);  // 2^-inf = 0 for masked keys
           S[i] = p;
           psum += p;
         }
@@ -780,10 +805,12 @@ __global__ __launch_bounds__(256, 2) void row_attention_prefill_bf16_kernel(
       psum += __shfl_xor(psum, 32, 64);
       l = l * corr + psum;
       mx = m_new;
+      if (__any(corr != 1.f)) {   // a running maximum moved somewhere in the wave
 #pragma unroll
-      for (int k = 0; k < DVB; ++k)
+        for (int k = 0; k < DVB; ++k)
 #pragma unroll
-        for (int i = 0; i < 16; ++i) acc[k][i] *= corr;
+          for (int i = 0; i < 16; ++i) acc[k][i] *= corr;
+      }
     }
     // ---- O^T += V_tile^T . P^T, three parts of p ---------------------------------
 #pragma unroll

@@ -38,6 +38,8 @@ def needed_extensions(cfg: ModelConfig, dtype: torch.dtype):
             names.append("_C")      # tuned GEMMs, grouped-GEMM experts
     else:
         names.append("_C")
+        if cfg.has_linear_layers:
+            names.append("_mix")    # recurrent layers' kernels
     return names
 
 
