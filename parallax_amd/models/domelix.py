@@ -151,6 +151,7 @@ class DomelixShardModel(nn.Module):
             self.norm = nn.Parameter(torch.empty(W), requires_grad=False)
             self.lm_head = ColumnParallelLinear(W, cfg.vocab_size)
         self.rope_cache = None  # the rotation's table is built per forward
+        self._side = None       # the experts' stream in decode steps
         # debugging aid: called with (global layer index, fp32 residual after
         # that layer) when set
         self.tap: Optional[Callable[[int, torch.Tensor], None]] = None
@@ -182,11 +183,23 @@ class DomelixShardModel(nn.Module):
         `pend` and are added by the kernel that writes the next layer's
         norms."""
         x = hidden.float().contiguous()
+        dev = x.device
         if self.is_last:
             dt = self.norm.dtype
         else:
             dt = self.layers[0].norm1.dtype if len(self.layers) else x.dtype
         pend = (None, None, None, None, 1.0, None)   # a, b, wa, wb, scale, f
+        # Decode steps: mixer and feed-forward do not read each other, so the
+        # experts run on a stream of their own beside the mixer (two branches
+        # of a captured graph). Every tensor that crosses is waited for before
+        # its owner lets go of it: h2 and f live until the streams have joined
+        # and the next layer's fork waits for the kernel that read f.
+        main = side = None
+        if x.is_cuda and not meta.is_prefill and self.graph_safe:
+            main = torch.cuda.current_stream(dev)
+            if self._side is None:
+                self._side = torch.cuda.Stream(dev)
+            side = self._side
 
         for i, layer in enumerate(self.layers):
             w2 = layer.norm2 if layer.mlp is not None else None
@@ -194,12 +207,22 @@ class DomelixShardModel(nn.Module):
                                               1.0, dt)
             if self.tap is not None and i > 0:
                 self.tap(self.start_layer + i - 1, x)
+            f = None
+            if layer.mlp is not None and side is not None:
+                side.wait_stream(main)
+                with torch.cuda.stream(side):
+                    f = layer.mlp(h2)
             if layer.kind == "parallel":
                 a, b = layer.mixer(h1, meta)
                 pend = (a, b, layer.left_out, layer.right_out, layer.half)
             else:
                 pend = (layer.mixer(h1, meta), None, None, None, 1.0)
-            pend += (layer.mlp(h2) if layer.mlp is not None else None,)
+            if layer.mlp is not None:
+                if side is not None:
+                    main.wait_stream(side)
+                else:
+                    f = layer.mlp(h2)
+            pend += (f,)
         w = self.norm if self.is_last else None
         out = x
         if w is not None or pend[0] is not None:

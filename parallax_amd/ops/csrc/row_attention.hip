@@ -486,7 +486,8 @@ DEVINL const T* ra_gate_row(const T* gate, int64_t gate_stride, int gate_w, int6
 // part layout: [T, H, splits, M, 2 + dv]: running max, denominator, sums
 // POOL false: no pooled rows exist, so the value loop has no per-key branch
 // and its loads of several keys are in flight together.
-template <typename T, int M, int HB, bool VEC, bool POOL>
+// REL: a distance bias or sinks are given.
+template <typename T, int M, int HB, bool VEC, bool POOL, bool REL>
 __global__ __launch_bounds__(256) void row_attention_kernel(
     T* __restrict__ out, float* __restrict__ out32, float* __restrict__ part,
     const float* __restrict__ q,
@@ -541,7 +542,7 @@ __global__ __launch_bounds__(256) void row_attention_kernel(
     hb[n] = sig ? head_bias[g * rep + min(r0 + n / M, rep - 1)] : 0.f;
     mx[n] = sig ? 0.f : -INFINITY;
     l[n] = 0.f;
-    if (sink != nullptr && split == 0 && wave == 0) {
+    if (REL && sink != nullptr && split == 0 && wave == 0) {
       mx[n] = sink[g * rep + min(r0 + n / M, rep - 1)];
       l[n] = 1.f;
     }
@@ -565,7 +566,7 @@ __global__ __launch_bounds__(256) void row_attention_kernel(
 #pragma unroll
     for (int n = 0; n < NQ; ++n) {
       s[n] = bv[n] = 0.f;
-      if (dist_bias != nullptr && valid)   // no pooled rows: key u is lo + u
+      if (REL && dist_bias != nullptr && valid)   // no pooled rows: key u is lo + u
         bv[n] = dist_bias[(int64_t)(g * rep + min(r0 + n / M, rep - 1)) * n_bias +
                           min(pos - lo - u, n_bias - 1)];
     }
@@ -604,7 +605,7 @@ __global__ __launch_bounds__(256) void row_attention_kernel(
     for (int n = 0; n < NQ; ++n) {
       float sc = s[n] * scale;
       if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
-      sc += bv[n];
+      if (REL) sc += bv[n];
       float p;
       if (sig) {
         p = valid ? ra_sigmoid(sc + hb[n]) : 0.f;
@@ -845,8 +846,8 @@ static void launch_ra_hb(const RaArgs& a) {
   const bool vec = (a.d % 8 == 0) && (a.dv % 8 == 0);
   int FL = 1;
   while (FL * 4 < a.dv) FL <<= 1;  // dv <= 256 -> FL <= 64
-#define RA_CALL(V, PL)                                                        \
-  hipLaunchKernelGGL((row_attention_kernel<T, M, HB, V, PL>), grid, dim3(256), shm, \
+#define RA_CALL(V, PL, RL)                                                    \
+  hipLaunchKernelGGL((row_attention_kernel<T, M, HB, V, PL, RL>), grid, dim3(256), shm, \
                      a.stream, (T*)a.out, a.out32, a.part, a.q,               \
                      (const T*)a.cache,                                       \
                      a.pool, a.block_tables, a.bt_stride, a.token_seq,        \
@@ -856,12 +857,16 @@ static void launch_ra_hb(const RaArgs& a) {
                      (const T*)a.gate, a.gate_stride, a.gate_w, a.vbase,      \
                      a.rot_cs, a.rot_inter, a.dist_bias, a.n_bias, a.sink)
   const bool pooled = a.pool != nullptr && a.window > 0 && a.P > 0;
-  if (vec) {
-    if (pooled) RA_CALL(true, true);
-    else RA_CALL(true, false);
+  const bool rel = M == 1 && !pooled && (a.dist_bias != nullptr || a.sink != nullptr);
+  if (rel) {
+    if (vec) RA_CALL(true, false, M == 1);
+    else RA_CALL(false, false, M == 1);
+  } else if (vec) {
+    if (pooled) RA_CALL(true, true, false);
+    else RA_CALL(true, false, false);
   } else {
-    if (pooled) RA_CALL(false, true);
-    else RA_CALL(false, false);
+    if (pooled) RA_CALL(false, true, false);
+    else RA_CALL(false, false, false);
   }
 #undef RA_CALL
   if (a.splits > 1)
