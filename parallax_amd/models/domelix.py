@@ -151,7 +151,7 @@ class DomelixShardModel(nn.Module):
             self.norm = nn.Parameter(torch.empty(W), requires_grad=False)
             self.lm_head = ColumnParallelLinear(W, cfg.vocab_size)
         self.rope_cache = None  # the rotation's table is built per forward
-        self._side = None       # the experts' stream in decode steps
+        self._side = None       # the experts' stream
         # debugging aid: called with (global layer index, fp32 residual after
         # that layer) when set
         self.tap: Optional[Callable[[int, torch.Tensor], None]] = None
@@ -189,13 +189,15 @@ class DomelixShardModel(nn.Module):
         else:
             dt = self.layers[0].norm1.dtype if len(self.layers) else x.dtype
         pend = (None, None, None, None, 1.0, None)   # a, b, wa, wb, scale, f
-        # Decode steps: mixer and feed-forward do not read each other, so the
-        # experts run on a stream of their own beside the mixer (two branches
-        # of a captured graph). Every tensor that crosses is waited for before
-        # its owner lets go of it: h2 and f live until the streams have joined
-        # and the next layer's fork waits for the kernel that read f.
+        # Mixer and feed-forward do not read each other, so the experts (grouped
+        # GEMMs) run on a stream of their own beside the mixer, whose recurrent
+        # kernels leave most of the chip idle; in a captured decode step they
+        # are two branches of the graph. Every tensor that crosses is waited
+        # for before its owner lets go of it: h2 and f live until the streams
+        # have joined, and the next layer's fork waits for the kernel that
+        # read f.
         main = side = None
-        if x.is_cuda and not meta.is_prefill and self.graph_safe:
+        if x.is_cuda and dt == torch.bfloat16 and self.graph_safe:
             main = torch.cuda.current_stream(dev)
             if self._side is None:
                 self._side = torch.cuda.Stream(dev)
