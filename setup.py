@@ -8,7 +8,7 @@ layer norm, sliding-window latent attention, gated linear attention, sandwich
 RMS norm, row-cache attention, post-norm residual step, minGRU, hyper-connected
 streams, matrix LSTM, softmax router, fixed-decay linear attention, gated delta
 rule, short convolution). Both are
-git-ignored; they travel to the GPU box with the gpurun snapshot.
+git-ignored and lie beside the sources.
 PARALLAX_EXT=_mix (or _C) builds one of them only.
 """
 

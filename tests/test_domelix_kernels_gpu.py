@@ -66,7 +66,7 @@ def test_parallel_rmsnorm_add(dtype, W):
 
 
 @pytest.mark.parametrize("dtype", BOTH)
-@pytest.mark.parametrize("H,dv", [(3, 20), (2, 33), (6, 32), (4, 128), (1, 256), (2, 300),
+@pytest.mark.parametrize("H,dv", [(3, 20), (2, 33), (6, 40), (4, 128), (1, 256), (2, 300),
                                   (32, 128), (33, 128), (5, 1)])
 @pytest.mark.parametrize("act", ["silu", "sigmoid"])
 def test_gated_rmsnorm(dtype, H, dv, act):
@@ -129,7 +129,7 @@ def test_rope_table():
 # (q/k heads, heads, key width, value width)
 SIZES = [(2, 2, 64, 64), (3, 3, 32, 40), (2, 4, 128, 128), (1, 3, 128, 72), (2, 2, 20, 12),
          (1, 2, 13, 7), (1, 1, 256, 96), (2, 2, 1, 1), (1, 1, 300, 20), (1, 1, 600, 8)]
-DECAYS = [0.9995, 0.6065306597126334, 0.0, 1.0]
+DECAYS = [0.9995, 0.55, 0.0, 1.0]
 
 
 def _sequences(short):
@@ -267,7 +267,7 @@ def _row_case(dtype, H, G, d, dv, lens, bs=16, seed=0):
 
 
 @pytest.mark.parametrize("dtype", BOTH)
-@pytest.mark.parametrize("H,G,d,dv", [(4, 1, 64, 64), (6, 2, 32, 48), (3, 3, 20, 12), (8, 2, 128, 128),
+@pytest.mark.parametrize("H,G,d,dv", [(8, 2, 64, 64), (6, 2, 32, 48), (3, 3, 20, 12), (8, 2, 128, 128),
                                       (5, 1, 7, 9), (2, 2, 64, 200)])
 @pytest.mark.parametrize("n_bias", [1, 9, 60, 1000])
 def test_row_attention_with_bias_sink_and_gate(dtype, H, G, d, dv, n_bias):
@@ -311,7 +311,7 @@ def test_row_attention_queries_that_are_no_bf16_numbers():
 
 
 @pytest.mark.parametrize("dtype", BOTH)
-@pytest.mark.parametrize("E,top,groups,keep", [(12, 3, 2, 1), (15, 4, 5, 2), (64, 8, 8, 3), (8, 8, 4, 4),
+@pytest.mark.parametrize("E,top,groups,keep", [(14, 3, 2, 1), (15, 4, 5, 2), (64, 8, 8, 3), (8, 8, 4, 4),
                                                (6, 1, 6, 1), (128, 6, 16, 4), (200, 5, 20, 7),
                                                (10, 4, 1, 1), (260, 4, 4, 2)])
 def test_route_softmax_in_groups(dtype, E, top, groups, keep):
